@@ -6,6 +6,8 @@ import dataclasses
 import torch
 import torch.nn as nn
 
+from ..ops.activation import softcap
+from ..ops.gemm import matmul_f32
 from ..ops.linear import LoraBranch, fused_linear
 from ..peft.lora import Linear4bit, LoraLayer, base_of
 from ..quant.int4 import Int4Linear, Int4Weight, int4_linear
@@ -299,6 +301,9 @@ class SeqBatch:
         self.len, self.pos = 0, None                                      # KVCache duck-typing (unused)
         self.cache_idx = desc[1].long()[desc[3].long()] * cache.max_len + desc[4].long()
         self.last = (desc[0][1:] - 1).long()
+        # a sequence that continues with more than one token: blocks of a kernel that split it over time must not
+        # read and write its carried rows in one launch
+        self.carried_runs = host is not None and any(p > 0 and b - a > 1 for p, a, b in zip(host[2], host[0], host[0][1:]))
 
     @classmethod
     def packed(cls, cache: "SeqStateCache", slots: list[int], lens: list[int], starts: list[int] | None = None):
@@ -465,6 +470,7 @@ class SeqStateCausalLM(nn.Module):
 
     config_class = None
     logit_scale = 1.0
+    logit_softcap = 0.0       # > 0: logits are bounded, softcap * tanh(logits / softcap)
 
     @classmethod
     def from_pretrained(cls, path: str, dtype=torch.bfloat16, device=None, **_):
@@ -482,15 +488,13 @@ class SeqStateCausalLM(nn.Module):
         return self.model.make_cache(batch, max_len, device)
 
     def compute_logits(self, h: torch.Tensor) -> torch.Tensor:
-        """Float logits ``head h * logit_scale`` (bf16 products accumulate in float and are not rounded back)."""
+        """Float logits ``head h * logit_scale``, bounded when ``logit_softcap`` is set (bf16 products accumulate in float and are not rounded back)."""
         w = self.lm_head.weight
-        h2 = h.reshape(-1, h.shape[-1])
-        if w.dtype == torch.float32 or not h2.is_cuda:
-            y = h2.float() @ w.float().t()
-        else:
-            y = torch.mm(h2, w.t(), out_dtype=torch.float32)
+        y = matmul_f32(h.reshape(-1, h.shape[-1]), w)
         if self.logit_scale != 1.0:
             y = y * self.logit_scale
+        if self.logit_softcap > 0:
+            y = softcap(y, self.logit_softcap)
         return y.view(*h.shape[:-1], w.shape[0])
 
     def forward(self, input_ids, attention_mask=None, labels=None, past_key_values=None, **_) -> CausalLMOutput:

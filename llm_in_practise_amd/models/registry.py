@@ -35,12 +35,18 @@ def _mamivik():
     return MamivikForCausalLM
 
 
+def _vefunex():
+    from .vefunex import VefunexForCausalLM
+    return VefunexForCausalLM
+
+
 REGISTRY = {
     "qwen3": _qwen, "qwen2": _qwen, "qwen3forcausallm": _qwen, "qwen2forcausallm": _qwen,
     "mobupel": _mobupel, "mobupelforcausallm": _mobupel,
     "dogudra": _dogudra, "dogudraforcausallm": _dogudra,
     "kitonex": _kitonex, "kitonexforcausallm": _kitonex,
     "mamivik": _mamivik, "mamivikforcausallm": _mamivik,
+    "vefunex": _vefunex, "vefunexforcausallm": _vefunex,
 }
 
 

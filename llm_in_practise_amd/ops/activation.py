@@ -76,13 +76,13 @@ def clipped_glu(z: torch.Tensor, limit: float) -> torch.Tensor:
     return ref.clipped_glu(z, limit)
 
 
-def silu_glu(z: torch.Tensor) -> torch.Tensor:
-    """``z = [gate | up]``: ``silu(gate) * up``."""
+def silu_glu(z: torch.Tensor, row_scale: torch.Tensor | None = None) -> torch.Tensor:
+    """``z = [gate | up]``: ``silu(gate) * up``; ``row_scale`` (float ``[T]``) multiplies gate and up first."""
     from . import reference as ref
     from ._native import native_seq, use_seq
     if use_seq(z):
-        return native_seq().ff_act(z.contiguous(), 2, 0.0)
-    return ref.silu_glu(z)
+        return native_seq().ff_act(z.contiguous(), 2, 0.0, row_scale)
+    return ref.silu_glu(z, row_scale)
 
 
 def gelu_glu(z: torch.Tensor) -> torch.Tensor:
@@ -102,3 +102,12 @@ def sigmoid_gate(y: torch.Tensor, gate_pre: torch.Tensor) -> torch.Tensor:
     if use_seq(y):
         return native_seq().sigmoid_gate(y, gate_pre)
     return ref.sigmoid_gate(y, gate_pre)
+
+
+def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """``cap * tanh(z / cap)`` of float logits, in place on the GPU."""
+    from . import reference as ref
+    from ._native import native_seq, use_seq
+    if use_seq(z):
+        return native_seq().softcap_(z, cap)
+    return ref.softcap(z, cap)

@@ -262,24 +262,27 @@ def qk_norm_store(u: torch.Tensor, nq: int, nk: int, q_weight: torch.Tensor, k_w
 
 def rope_kv_store(u: torch.Tensor, nq: int, nk: int, heads: int, kv_heads: int, inv_freq: torch.Tensor, rot_dims: int,
                   k_cache: torch.Tensor, v_cache: torch.Tensor, sb, half: bool = True, mag: float = 1.0,
-                  values_are_keys: bool = False) -> torch.Tensor:
+                  values_are_keys: bool = False, temp: tuple | None = None, v_eps: float | None = None) -> torch.Tensor:
     """The step's ``[q | k (| v)]`` rows ``u`` on their way into rotary attention: the first ``rot_dims`` entries of
     every q and k head are rotated at the token's position (``half``: entries ``i, i + rot_dims/2`` form a pair, else
     neighbours; ``mag`` multiplies sine and cosine); the rotated k goes to ``k_cache`` ``[slots, max_len, nk]`` at each
     token's slot and position; ``v_cache`` gets ``u``'s v columns or, with ``values_are_keys``, the k columns as they
-    came (unrotated).  Angles and the rotation are float.  Returns the rotated q ``[T, nq]``."""
+    came (unrotated).  Angles and the rotation are float.  Returns the rotated q ``[T, nq]``.  ``temp = (coef, every)``:
+    q at position ``p`` is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``.  ``v_eps``: each kv head's value
+    is divided by its root mean square (that eps inside the root) before it is cached.  ``rot_dims = 0``: no rotation."""
     from ._native import native_seq, use_seq
     if use_seq(u):
         return native_seq().rope_kv_store(u, nq, nk, heads, kv_heads, inv_freq, rot_dims, k_cache, v_cache, sb.desc, half,
-                                          mag, values_are_keys)
+                                          mag, values_are_keys, *(temp or (0.0, 0)), -1.0 if v_eps is None else v_eps)
     return ref.rope_kv_store(u, nq, nk, heads, kv_heads, inv_freq, rot_dims, k_cache, v_cache, sb, half, mag,
-                             values_are_keys)
+                             values_are_keys, temp, v_eps)
 
 
 def biased_attention(q, k_cache, v_cache, bias: torch.Tensor | None, heads: int, kv_heads: int, scale: float, sb,
                      block: int = 0, sink: float | torch.Tensor | None = None, nsplit: int = 1, window: int = 0,
-                     out: torch.Tensor | None = None, out_scale: float = 1.0):
-    """Causal grouped-query softmax attention over a slot-indexed cache with three optional parts:
+                     out: torch.Tensor | None = None, out_scale: float = 1.0, softcap: float = 0.0,
+                     gate: torch.Tensor | None = None):
+    """Causal grouped-query softmax attention over a slot-indexed cache with optional parts:
     ``bias`` float ``[H, ND]`` adds ``bias[h, min(i - j, ND - 1)]`` to the scaled score of query ``i`` and key ``j``
     (``scale`` does not multiply it); ``block > 0`` lets a query see only keys of its own run of ``block`` positions
     (runs counted from the sequence's position 0); ``sink`` adds one key of that score and no value to every
@@ -288,11 +291,14 @@ def biased_attention(q, k_cache, v_cache, bias: torch.Tensor | None, heads: int,
     float.  ``nsplit`` cuts each query's keys into that many independent sweeps (decode).  ``sink`` may be a float
     tensor ``[H]``: one score per head.  ``window > 0``: a query sees only the keys less than ``window`` positions
     back (itself included).  ``out`` (``[T, H*dv]``, a column slice of a wider matrix is fine) receives the result,
-    multiplied by ``out_scale``."""
+    multiplied by ``out_scale``.  ``softcap > 0``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` (before
+    a bias; a sink is not capped).  ``gate`` ``[T, H*dv]`` (a column slice is fine): the result is multiplied element by
+    element with its sigmoid."""
     from ._native import native_seq, use_seq
     if use_seq(q):
         per_head = sink if torch.is_tensor(sink) else None
         return native_seq().biased_attention(q, k_cache, v_cache, bias, heads, kv_heads, scale, block,
                                              sink is not None, 0.0 if per_head is not None else float(sink or 0.0),
-                                             nsplit, sb.desc, sb.tiles, window, per_head, out, out_scale)
-    return ref.biased_attention(q, k_cache, v_cache, bias, heads, kv_heads, scale, block, sink, sb, window, out, out_scale)
+                                             nsplit, sb.desc, sb.tiles, window, per_head, out, out_scale, softcap, gate)
+    return ref.biased_attention(q, k_cache, v_cache, bias, heads, kv_heads, scale, block, sink, sb, window, out, out_scale,
+                                softcap, gate)

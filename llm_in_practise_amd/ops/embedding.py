@@ -123,17 +123,19 @@ def embed_sincos(tokens: torch.Tensor, positions: torch.Tensor, table: torch.Ten
 
 
 def embed_pair(tokens: torch.Tensor, table: torch.Tensor, pair_table: torch.Tensor | None, prev: torch.Tensor | None,
-               scale: float, mul_prev: int, mul_cur: int, sb):
+               scale: float, mul_prev: int, mul_cur: int, sb, out: torch.Tensor | None = None):
     """Scaled token embedding plus a hashed embedding of the (previous, current) token pair: row
     ``(prev*mul_prev + cur*mul_cur) mod buckets`` of ``pair_table`` ``[buckets + 1, W]``; a sequence's first token
     takes the extra last row.  ``prev`` (int32 ``[slots]``) carries each sequence's last token from step to step
-    and is updated in place.  Returns ``(x float [T, W], x in the table's dtype)``."""
+    and is updated in place.  Returns ``(x float [T, W], x in the table's dtype)``.  ``out`` (float ``[T, W]``,
+    contiguous) receives ``x``; no second copy is made then (``None`` is returned for it)."""
     from . import reference as ref
     from ._native import native_seq, use_seq
     if use_seq(table):
         return tuple(native_seq().embed_pair(tokens.reshape(-1).long().contiguous(), table, pair_table, prev, scale,
-                                             mul_prev, mul_cur, sb.desc, sb.live))
-    return ref.embed_pair(tokens, table, pair_table, prev, scale, mul_prev, mul_cur, sb)
+                                             mul_prev, mul_cur, sb.desc, sb.live, out))
+    x, h = ref.embed_pair(tokens, table, pair_table, prev, scale, mul_prev, mul_cur, sb)
+    return (x, h) if out is None else (out.copy_(x), None)
 
 
 def embed_learned(tokens: torch.Tensor, positions: torch.Tensor, table: torch.Tensor, pos_table: torch.Tensor,

@@ -210,3 +210,11 @@ def _base_gemm_t(dy, base, ext_a=None, ext_b=None, c=None):
         base = _nf4_dequant_bf16(base) if (base.kernel_ok() and dy.is_cuda) else dequantize_nf4(base, dy.dtype)
     dx = _dense_dx(dy, base, c)
     return dx if ext_a is None else dx.addmm_(ext_a, ext_b.t())
+
+
+def matmul_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """``x w^T`` with a float result (``x`` ``[T, K]`` and ``w`` ``[N, K]`` of one dtype): bf16 operands accumulate in
+    float and the sums are not rounded back (logits, pre-activations of recurrences)."""
+    if x.dtype == torch.float32 or not x.is_cuda:
+        return x.float() @ w.float().t()
+    return torch.mm(x, w.t(), out_dtype=torch.float32)

@@ -190,7 +190,8 @@ PAD_ROWS = 128      # sorted path: an expert's products run over a multiple of t
 
 def moe_glu_experts(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor,
                     weights: torch.Tensor, limit: float, shared: torch.Tensor | None = None,
-                    few_tokens: bool = False, act: str = "clipped", shared_gate: torch.Tensor | None = None) -> torch.Tensor:
+                    few_tokens: bool = False, act: str = "clipped", shared_gate: torch.Tensor | None = None,
+                    weight_input: bool = False) -> torch.Tensor:
     """Weighted sum of the chosen GLU experts' outputs, float ``[T, W]`` (``act="clipped"``: the clipped GLU with
     ``limit``; ``act="silu"``: ``silu(gate) * up``, ``limit`` unused; ``shared_gate`` float ``[T]``: the shared
     expert's output is multiplied by its sigmoid).  ``w_gate_up`` ``[E, 2, F, W]``,
@@ -198,19 +199,24 @@ def moe_glu_experts(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tens
     added.  ``few_tokens`` (decode steps, captured graphs): every (token, expert) pair streams its expert's rows in
     two kernels with no sort and no host round trip.  Otherwise rows are sorted by expert, every expert runs one
     vendor matrix product pair over its run of rows (one host read of the run lengths; long runs are rounded up to a
-    multiple of ``PAD_ROWS`` rows), and a kernel combines."""
+    multiple of ``PAD_ROWS`` rows), and a kernel combines.  ``weight_input`` (``act="silu"``): a pair's weight multiplies
+    the expert's input instead of its output, ``sum_e expert_e(w_e h)``; it is applied in float to the gate and up
+    products, which are linear in the input."""
     from . import reference as ref
     from ._native import native_seq, use_seq
     from .activation import clipped_glu, silu_glu
     if act not in ("clipped", "silu"):
         raise ValueError(f"experts: unknown activation {act!r}")
     mode = 1 if act == "clipped" else 2
-    glu = (lambda z: clipped_glu(z, limit)) if mode == 1 else silu_glu
+    if weight_input and mode != 2:
+        raise ValueError("experts: input weights go with the SiLU activation")
+    glu = (lambda z, s: clipped_glu(z, limit)) if mode == 1 else silu_glu
     T, W = h.shape
     E, _, F_, _ = w_gate_up.shape
     top = idx.shape[1]
     if use_seq(h) and few_tokens:
-        return native_seq().moe_pairs(h.contiguous(), w_gate_up, w_down, idx, weights, shared, limit, mode, shared_gate)
+        return native_seq().moe_pairs(h.contiguous(), w_gate_up, w_down, idx, weights, shared, limit, mode, shared_gate,
+                                      weight_input)
     flat = idx.reshape(-1).long()
     order = torch.sort(flat, stable=True).indices
     counts = torch.bincount(flat, minlength=E).tolist()[:E]
@@ -223,12 +229,17 @@ def moe_glu_experts(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tens
     torch.index_select(h, 0, (order // top)[:rows], out=xs[:rows])
     xs[rows:].zero_()
     ys = torch.empty(rows + pad, W, dtype=h.dtype, device=h.device)
+    ws = None
+    if weight_input:
+        ws = weights.new_zeros(rows + pad)
+        torch.index_select(weights.reshape(-1), 0, order[:rows], out=ws[:rows])
+        weights = torch.ones_like(weights)
     a = 0
     for e, n in enumerate(counts):
         if n:
             m = min(-(-n // pad) * pad, rows + pad - a) if pad else n
             z = xs[a:a + m] @ w_gate_up[e].reshape(2 * F_, W).t()
-            torch.mm(glu(z), w_down[e].t(), out=ys[a:a + m])
+            torch.mm(glu(z, None if ws is None else ws[a:a + m]), w_down[e].t(), out=ys[a:a + m])
             a += n
     pos = torch.empty_like(order)
     pos[order] = torch.arange(order.numel(), device=order.device)

@@ -145,18 +145,21 @@ def dual_norm_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch
 
 def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate_pre: torch.Tensor, eps: float,
                    den: torch.Tensor | None = None, floor: torch.Tensor | None = None,
-                   out: torch.Tensor | None = None, scale: float = 1.0) -> torch.Tensor:
+                   out: torch.Tensor | None = None, scale: float = 1.0, act: str = "sigmoid") -> torch.Tensor:
     """Read-out of a recurrent mixer: ``o`` float ``[T, H, dv]`` is RMS-normed per head, scaled by ``weight``
-    (``[dv]`` shared by the heads or ``[H * dv]``) and multiplied by ``sigmoid(gate_pre)``; returns ``[T, H * dv]``
+    (``[dv]`` shared by the heads or ``[H * dv]``) and multiplied by ``act(gate_pre)`` (``"sigmoid"`` or ``"silu"``);
+    returns ``[T, H * dv]``
     in ``gate_pre``'s dtype.  With ``den`` / ``floor`` (float ``[T, H]``) ``o`` is first divided by
     ``max(|den|, floor) + 1e-6`` (the mLSTM's normaliser).  ``out`` (``[T, H * dv]``, a column slice of a wider matrix
     is fine) receives the result, multiplied by ``scale``."""
     from ._native import native_seq, use_seq
+    if act not in ("sigmoid", "silu"):
+        raise ValueError(f"head_norm_gate: unknown gate activation {act!r}")
     if use_seq(o):
-        return native_seq().head_norm_gate(o, weight, gate_pre, eps, den, floor, out, scale)
+        return native_seq().head_norm_gate(o, weight, gate_pre, eps, den, floor, out, scale, act == "silu")
     if den is not None:
         o = o / (torch.maximum(den.abs(), floor) + 1e-6)[..., None]
-    return ref.head_norm_gate(o, weight, gate_pre, eps, out, scale)
+    return ref.head_norm_gate(o, weight, gate_pre, eps, out, scale, act == "silu")
 
 
 def scaled_postnorm(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, alpha: float, eps: float,
@@ -197,3 +200,29 @@ def hyper_mix_norm(X: torch.Tensor, y: torch.Tensor | None, mix: torch.Tensor | 
     if use_seq(X):
         return native_seq().hyper_mix_norm(X, y, mix, out, read, weight, eps, dtype == torch.bfloat16)
     return ref.hyper_mix_norm(X, y, mix, out, read, weight, eps, dtype)
+
+
+def residual_dyt(x: torch.Tensor, y: torch.Tensor | None, mult: float, weight: torch.Tensor, bias: torch.Tensor,
+                 alpha: float, dtype: torch.dtype, conv: torch.Tensor | None = None, state: torch.Tensor | None = None,
+                 streams: torch.Tensor | None = None, n: int = 0, depth: torch.Tensor | None = None, sb=None):
+    """A sublayer's exit and the next one's entry for a residual block with Dynamic-Tanh norms, all in one kernel:
+
+    * ``r = x + mult * y`` (``x`` float ``[T, W]``, ``y`` float or the activation dtype; ``y = None``: ``r = x``);
+    * with ``depth`` (float ``[n + 1]``) the end of layer ``n - 1``: ``r`` is kept as ``streams[n]`` (``streams`` float
+      ``[layers + 1, T, W]``, entry 0 the embedding output) and replaced by ``sum_j depth[j] * streams[j]``, j <= n;
+    * ``h = tanh(alpha * r) * weight + bias``;
+    * with ``conv`` (float ``[taps, W]``) ``h_t + sum_j conv[j] h_(t - taps + 1 + j)`` per channel, zeros before a
+      sequence's start; ``state`` float ``[slots, taps - 1, W]`` carries the last ``h`` of every sequence from step to
+      step, in place.
+
+    Returns ``(r, h in dtype)``.  ``x`` is not written: the convolution's neighbours recompute each other's ``h``."""
+    from ._native import native_seq, use_seq
+    if use_seq(x):
+        desc = sb.desc if sb is not None else []
+        tiles, live = (sb.tiles, sb.live) if sb is not None else ([], None)
+        old = state
+        if conv is not None and state is not None and sb.carried_runs:
+            old = state.clone()      # several blocks of one sequence: the carried rows are read by one, written by another
+        return tuple(native_seq().residual_dyt(x, y, mult, weight, bias, alpha, dtype == torch.bfloat16, conv, state, old,
+                                               streams, n, depth, desc, live, tiles))
+    return ref.residual_dyt(x, y, mult, weight, bias, alpha, dtype, conv, state, streams, n, depth, sb)

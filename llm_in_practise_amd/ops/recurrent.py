@@ -5,8 +5,10 @@
 * :func:`general_delta_scan` — the delta rule with separate decay, removal and write vectors (both the decay and
   the removal read the old state).
 * :func:`ssd_scan` — a selective state space in its state-space-duality form (scalar decay and step size per head).
+* :func:`selective_scan` — a selective state space with a step size per channel and a decay per (channel, state).
+* :func:`gated_linear_scan` — linear attention with a data-dependent decay per key channel.
 
-All keep ``S`` as ``[slots, H, dv, dk]`` float (one column of the ``[dk, dv]`` matrix contiguous), read
+All but :func:`selective_scan` (``[slots, channels, states]``) keep ``S`` as ``[slots, H, dv, dk]`` float (one column of the ``[dk, dv]`` matrix contiguous), read
 and write it in place, and treat a sequence that starts at position 0 as starting from zero state.  The same kernel
 serves prefill (a scan over the step's tokens with the state in registers) and decode (one token: load, update,
 store).  HIP kernels: csrc/kernels/seq/seq_scan.hip; the CPU path is ops/reference.py.
@@ -81,3 +83,25 @@ def general_delta_scan(r, k, v, w, a, kinv, S, heads: int, sb):
     if use_seq(r):
         return native_seq().general_delta_scan(r, k, v, w, a, kinv, S, heads, sb.desc, sb.live)
     return ref.general_delta_scan(r, k, v, w, a, kinv, S, heads, sb)
+
+
+def selective_scan(x, dt_pre, dt_bias, b, c, a_log, d_skip, z, S, sb, out=None, scale: float = 1.0):
+    """Selective state space (Mamba), per channel ``c`` and state ``n``: ``dt = softplus(dt_pre + dt_bias)``,
+    ``S[c, n] <- exp(-dt_c exp(a_log[c, n])) S[c, n] + dt_c x_c b_n``, ``y_c = sum_n S[c, n] c_n + d_skip_c x_c``; returns
+    ``scale * y * silu(z)``.  ``x, z`` ``[T, C]`` and ``b, c`` ``[T, N]`` in the activation dtype (column slices are fine),
+    ``dt_pre`` float ``[T, C]``, ``a_log`` float ``[C, N]``, ``dt_bias, d_skip`` float ``[C]``; ``S`` float
+    ``[slots, C, N]`` in place.  Step sizes, decays, the state and the gate are float.  ``out`` (``[T, C]``, a column
+    slice of a wider matrix is fine) receives the result."""
+    if use_seq(x):
+        return native_seq().selective_scan(x, dt_pre, dt_bias, b, c, a_log, d_skip, z, S, sb.desc, sb.live, out, scale)
+    return ref.selective_scan(x, dt_pre, dt_bias, b, c, a_log, d_skip, z, S, sb, out, scale)
+
+
+def gated_linear_scan(q, k, v, z, z_bias, tau: float, q_scale: float, S, heads: int, sb):
+    """Gated linear attention, per head with ``S`` ``[dk, dv]``: ``S <- diag(a) S + k v^T``, ``o = q_scale S^T q`` with
+    ``a = sigmoid(z + z_bias)^(1 / tau)``.  ``q, k`` ``[T, H*dk]``, ``v`` ``[T, H*dv]`` in the activation dtype, ``z``
+    float ``[T, H*dk]``, ``z_bias`` float ``[H*dk]``; ``S`` float ``[slots, H, dv, dk]`` in place.  Decays and the state are
+    float (the decay as ``exp(log sigmoid / tau)``).  Returns float ``[T, H, dv]``."""
+    if use_seq(q):
+        return native_seq().gated_linear_scan(q, k, v, z, z_bias, tau, q_scale, S, heads, sb.desc, sb.live)
+    return ref.gated_linear_scan(q, k, v, z, z_bias, tau, q_scale, S, heads, sb)

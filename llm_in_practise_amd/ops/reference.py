@@ -183,10 +183,10 @@ def polynorm(z, coef, eps: float):
     return out.to(z.dtype)
 
 
-def head_norm_gate(o, w, gate, eps: float, out=None, scale: float = 1.0):
+def head_norm_gate(o, w, gate, eps: float, out=None, scale: float = 1.0, silu: bool = False):
     T, H, dv = o.shape
     y = _unit_rms(o, eps) * (w.view(H, dv) if w.numel() != dv else w)
-    y = y.reshape(T, H * dv) * torch.sigmoid(gate.float()) * scale
+    y = y.reshape(T, H * dv) * (F.silu(gate.float()) if silu else torch.sigmoid(gate.float())) * scale
     if out is None:
         return y.to(gate.dtype)
     out.copy_(y)
@@ -479,7 +479,7 @@ def qk_norm_store(u, nq: int, nk: int, qw, kw, kc, vc, v_first, lam, eps: float,
 
 
 def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, sink, sb, window: int = 0, out=None,
-                     out_scale: float = 1.0):
+                     out_scale: float = 1.0, softcap: float = 0.0, gate=None):
     T = q.shape[0]
     dk, dv = q.shape[1] // H, vc.shape[2] // G
     rep = H // G
@@ -491,6 +491,8 @@ def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, 
         kk = kc[slot, :L].float().view(L, G, dk).repeat_interleave(rep, 1)      # [L, H, dk]
         vv = vc[slot, :L].float().view(L, G, dv).repeat_interleave(rep, 1)
         sc = torch.einsum("thd,lhd->htl", q[a:e].float().view(e - a, H, dk), kk) * scale
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
         qp = pos0[b] + torch.arange(e - a, device=q.device)
         kp = torch.arange(L, device=q.device)
         dist = qp[:, None] - kp[None, :]
@@ -503,6 +505,8 @@ def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, 
             sc = sc + bias[:, dist.clamp(0, bias.shape[1] - 1)]
         w = _softmax_with_sink(sc.masked_fill(~vis[None], float("-inf")), sink)
         res[a:e] = torch.einsum("htl,lhd->thd", w, vv).reshape(e - a, H * dv)
+    if gate is not None:
+        res = res * torch.sigmoid(gate.float())
     if out_scale != 1.0:
         res = res * out_scale
     if out is None:
@@ -528,20 +532,28 @@ def route_scored(z, corr, top: int, groups: int, keep: int, scale: float, sigmoi
     return idx.int(), w * scale
 
 
-def silu_glu(z):
+def silu_glu(z, row_scale=None):
     F_ = z.shape[-1] // 2
-    return (F.silu(z[..., :F_].float()) * z[..., F_:].float()).to(z.dtype)
+    g, u = z[..., :F_].float(), z[..., F_:].float()
+    if row_scale is not None:
+        g, u = g * row_scale[:, None], u * row_scale[:, None]
+    return (F.silu(g) * u).to(z.dtype)
 
 
 # ---- sliding-window attention whose values are its keys, generalised delta rule, GELU GLU, element-wise output gate
 def rope_kv_store(u, nq: int, nk: int, H: int, G: int, inv_freq, dims: int, kc, vc, sb, half: bool, mag: float,
-                  values_are_keys: bool):
+                  values_are_keys: bool, temp=None, v_eps=None):
     T = u.shape[0]
     dk = nq // H
     pos = sb.desc[4]
-    q = rotate(u[:, :nq].float().view(T, H, dk), pos, inv_freq, dims, half, mag).reshape(T, nq).to(u.dtype)
+    q = rotate(u[:, :nq].float().view(T, H, dk), pos, inv_freq, dims, half, mag).reshape(T, nq)
+    if temp is not None:
+        q = q * (1.0 + temp[0] * torch.log((torch.div(pos + 1, int(temp[1]), rounding_mode="floor") + 1).float()))[:, None]
+    q = q.to(u.dtype)
     k = rotate(u[:, nq:nq + nk].float().view(T, G, dk), pos, inv_freq, dims, half, mag).reshape(T, nk)
     v = u[:, nq:nq + nk] if values_are_keys else u[:, nq + nk:]
+    if v_eps is not None:
+        v = _unit_rms(v.float().reshape(T, G, -1), v_eps).reshape(T, -1)
     kc.view(-1, nk).index_copy_(0, sb.cache_idx, k.to(kc.dtype))
     vc.view(-1, vc.shape[2]).index_copy_(0, sb.cache_idx, v.to(vc.dtype))
     return q
@@ -583,3 +595,73 @@ def gelu_glu(z):
 
 def sigmoid_gate(y, gate):
     return (y.float() * torch.sigmoid(gate.float())).to(y.dtype)
+
+
+# ---- Dynamic-Tanh pre-norm with an input convolution over a depth-averaged residual; selective scan with a step per
+# channel; gated linear attention
+def residual_dyt(x, y, mult: float, weight, bias, alpha: float, dtype, conv=None, state=None, streams=None, n: int = 0,
+                 depth=None, sb=None):
+    r = x if y is None else x + mult * y.float()
+    if depth is not None:
+        streams[n] = r
+        r = (depth[:, None, None] * streams[:n + 1]).sum(0)
+    h = torch.tanh(alpha * r) * weight + bias
+    if conv is not None:
+        taps = conv.shape[0]
+        off, slots, pos0 = sb.host()
+        out = torch.empty_like(h)
+        for b, slot in enumerate(slots):
+            a, e = off[b], off[b + 1]
+            prev = h.new_zeros(0, h.shape[1])
+            if taps > 1:
+                prev = state[slot].clone() if pos0[b] > 0 else h.new_zeros(taps - 1, h.shape[1])
+            ext = torch.cat([prev, h[a:e]], 0)
+            if taps > 1 and sb.is_live(b):
+                state[slot] = ext[-(taps - 1):]
+            out[a:e] = h[a:e] + sum(conv[j] * ext[j:j + e - a] for j in range(taps))
+        h = out
+    return r, h.to(dtype)
+
+
+def selective_scan(x, dt_pre, dt_bias, b, c, a_log, d_skip, z, S, sb, out=None, scale: float = 1.0):
+    T, C = x.shape
+    xf, bf, cf = x.float(), b.float(), c.float()
+    dt = F.softplus(dt_pre.float() + dt_bias)
+    A = -torch.exp(a_log)
+    y = torch.zeros(T, C, dtype=torch.float32, device=x.device)
+    off, slots, pos0 = sb.host()
+    for i, slot in enumerate(slots):
+        if not sb.is_live(i):
+            continue
+        s = torch.zeros_like(S[slot]) if pos0[i] == 0 else S[slot].clone()   # [C, N]
+        for t in range(off[i], off[i + 1]):
+            s = torch.exp(dt[t][:, None] * A) * s + (dt[t] * xf[t])[:, None] * bf[t][None, :]
+            y[t] = (s * cf[t][None, :]).sum(-1) + d_skip * xf[t]
+        S[slot] = s
+    y = y * F.silu(z.float()) * scale
+    if out is None:
+        return y.to(x.dtype)
+    out.copy_(y)
+    return out
+
+
+def gated_linear_scan(q, k, v, z, z_bias, tau: float, q_scale: float, S, H: int, sb):
+    T = q.shape[0]
+    dk, dv = q.shape[1] // H, v.shape[1] // H
+    qf, kf, vf = q.float().view(T, H, dk) * q_scale, k.float().view(T, H, dk), v.float().view(T, H, dv)
+    g = torch.exp(F.logsigmoid(z.float() + z_bias) / tau).view(T, H, dk)
+    out = torch.zeros(T, H, dv, dtype=torch.float32, device=q.device)
+    off, slots, pos0 = sb.host()
+    for b, slot in enumerate(slots):
+        if not sb.is_live(b):
+            continue
+        s = torch.zeros_like(S[slot]) if pos0[b] == 0 else S[slot].clone()   # [H, dv, dk]
+        for t in range(off[b], off[b + 1]):
+            s = s * g[t][:, None, :] + vf[t][:, :, None] * kf[t][:, None, :]
+            out[t] = (s * qf[t][:, None, :]).sum(-1)
+        S[slot] = s
+    return out
+
+
+def softcap(z, cap: float):
+    return cap * torch.tanh(z / cap)
