@@ -15,7 +15,8 @@
 // sequence's position 0), a sliding window (a query sees only the keys less than `window` positions back, itself
 // included), and a sink (one more key of a fixed score, or of a learned score per head, without a value in every
 // softmax).  With one key split the matrix-core sweep normalises and writes the activation type itself; otherwise
-// k_gqa_merge does.  The output may be a column slice of a wider matrix (row stride ldo) and is multiplied by
+// k_gqa_merge does.  Scores may be bounded (softcap * tanh(score / softcap)), the result may be multiplied element by
+// element with the sigmoid of a gate.  The output may be a column slice of a wider matrix (row stride ldo) and is multiplied by
 // out_scale.
 #include "seq_common.h"
 
@@ -33,6 +34,9 @@ struct GqaExtra {
   const float* sinks;  // [H] or null: a sink score per head, in place of sink_logit
   int ldo;             // row stride of out
   float out_scale;
+  float softcap;       // 0: plain scores
+  const void* gate;    // [T, H * dv] gate pre-activations in the activation type or null; rows ldg apart (8-byte rows)
+  int ldg;
 };
 
 constexpr int MAXC = 16;   // value columns per lane: G * dv <= 64 * MAXC
@@ -67,6 +71,7 @@ __global__ __launch_bounds__(64) void k_talk_attn_partial(const T* __restrict__ 
       float a = 0.f;
       for (int i = 0; i < dk; ++i) a += sq[i] * (float)kr[i];
       sc = a * scale;
+      if (GQA && x.softcap > 0.f) sc = x.softcap * tanhf(sc / x.softcap);
       if (GQA && x.bias != nullptr) sc += x.bias[(size_t)g * x.nd + min(p - j, x.nd - 1)];
     }
     const float mn = fmaxf(m, wave_max(sc));
@@ -151,6 +156,8 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
   // p0 - jb - 31 + i: lane i fetches that one bias and the 16 a lane needs come from its neighbours' registers
   const int p0 = HEADS ? pos_q : d.tok_pos[t0];
   const float sl2 = scale * 1.4426950408889634f;   // scores in units of log2: v_exp_f32 is 2^x
+  // bounded scores: cap tanh(u) = cap - 2 cap / (e^2u + 1), with e^2u as a power of two
+  const float cap = GQA ? x.softcap : 0.f, cl2 = cap * 1.4426950408889634f, ce = cap > 0.f ? 2.f * sl2 / cap : 0.f;
   const int trow = 4 * (lane >> 5) + ((lane & 15) >> 2), tcol = 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
   const int per = (pmax - lo_t + nsplit) / nsplit, j0 = lo_t + z * per, j1 = min(pmax + 1, j0 + per);
   const bf16* kbase = kc + ((size_t)slot * max_len) * ldk + kh * dk + 8 * hi;
@@ -222,6 +229,7 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
       const int kk = (r & 3) + 8 * (r >> 2) + 4 * hi, key = jb + kk;
       const bool seen = key <= pos_q && key < j1 && (!GQA || key >= lo_q);
       float v = sc[r] * sl2;
+      if (GQA && cap > 0.f) v = cl2 - 2.f * cl2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[r] * ce) + 1.f);
       if (GQA && !HEADS && brow != nullptr) v += __shfl(bw, ql - kk + 31, 64);
       if (GQA && HEADS && brow != nullptr && seen) v += brow[min(pos_q - key, x.nd - 1)] * 1.4426950408889634f;
       sc[r] = seen ? v : -INFINITY;
@@ -268,6 +276,18 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
     const float den = l * e + (x.sink ? __builtin_amdgcn_exp2f(sk - mf) : 0.f);
     const float inv = den > 0.f ? e / den * x.out_scale : 0.f;
     bf16* orow = (bf16*)x.out + (size_t)tq * x.ldo + g * dv;
+    if (x.gate != nullptr) {
+      const bf16* grow = (const bf16*)x.gate + (size_t)tq * x.ldg + g * dv;
+#pragma unroll
+      for (int dt = 0; dt < NDT; ++dt)
+        if (dt < ndt)
+#pragma unroll
+          for (int r4 = 0; r4 < 4; ++r4) {
+            const bf16x4 gv = *reinterpret_cast<const bf16x4*>(grow + dt * 32 + 8 * r4 + 4 * hi);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[dt][4 * r4 + j] *= sigmoidf_((float)gv[j]);
+          }
+    }
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt)
       if (dt < ndt)
@@ -388,7 +408,7 @@ void seq_attn_sweep(int code, const void* q, int ldq, const void* kc, int ldk, c
                     float* pl, float* pu, int H, int G, int dk, int dv, int max_len, int nsplit, float scale,
                     const int* tile_seq, const int* tile_t0, int ntiles, SeqDesc d, hipStream_t st) {
   sweep<false>(code, q, ldq, kc, ldk, vc, ldv, pm, pl, pu, H, G, dk, dv, max_len, nsplit, scale, tile_seq, tile_t0,
-               ntiles, d, GqaExtra{nullptr, 0, 0, 0, 0.f, nullptr, 0, nullptr, 0, 1.f}, st);
+               ntiles, d, GqaExtra{nullptr, 0, 0, 0, 0.f, nullptr, 0, nullptr, 0, 1.f, 0.f, nullptr, 0}, st);
 }
 
 // Merge of a GQA sweep's key splits: one wave per (token, head); the sink joins the denominator here.
@@ -396,7 +416,8 @@ template <typename T>
 __global__ __launch_bounds__(64) void k_gqa_merge(const float* __restrict__ pm, const float* __restrict__ pl,
                                                   const float* __restrict__ pu, T* __restrict__ out, int H, int dv,
                                                   int nsplit, int sink, float sink_logit,
-                                                  const float* __restrict__ sinks, int ldo, float out_scale) {
+                                                  const float* __restrict__ sinks, int ldo, float out_scale,
+                                                  const T* __restrict__ gate, int ldg) {
   const int t = blockIdx.x, g = blockIdx.y, lane = threadIdx.x;
   const size_t b = ((size_t)t * H + g) * nsplit;
   if (sinks != nullptr) sink_logit = sinks[g];
@@ -409,6 +430,7 @@ __global__ __launch_bounds__(64) void k_gqa_merge(const float* __restrict__ pm, 
     float u = 0.f;
     for (int z = 0; z < nsplit; ++z)
       if (pm[b + z] != -INFINITY) u += expf(pm[b + z] - mx) * pu[(b + z) * dv + col];
+    if (gate != nullptr) u *= sigmoidf_((float)gate[(size_t)t * ldg + g * dv + col]);
     out[(size_t)t * ldo + g * dv + col] = (T)(u * inv);
   }
 }
@@ -418,16 +440,17 @@ __global__ __launch_bounds__(64) void k_gqa_merge(const float* __restrict__ pm, 
 // with G = 1); the output rows are ldo elements apart.
 void seq_gqa_attention(int code, const void* q, int ldq, const void* kc, int ldk, const void* vc, int ldv, float* pm,
                        float* pl, float* pu, const float* bias, int nd, int block, int window, int sink, float sink_logit,
-                       const float* sinks, void* out, int ldo, float out_scale, int H, int G, int dk, int dv, int max_len,
-                       int nsplit, float scale, const int* tile_seq, const int* tile_t0, int ntiles, SeqDesc d,
-                       hipStream_t st) {
+                       const float* sinks, void* out, int ldo, float out_scale, float softcap, const void* gate, int ldg,
+                       int H, int G, int dk, int dv, int max_len, int nsplit, float scale, const int* tile_seq,
+                       const int* tile_t0, int ntiles, SeqDesc d, hipStream_t st) {
   if (d.Ttot == 0) return;
   const bool direct = sweep<true>(code, q, ldq, kc, ldk, vc, ldv, pm, pl, pu, H, G, dk, dv, max_len, nsplit, scale,
                                   tile_seq, tile_t0, ntiles, d,
-                                  GqaExtra{bias, nd, block, sink, sink_logit, out, window, sinks, ldo, out_scale}, st);
+                                  GqaExtra{bias, nd, block, sink, sink_logit, out, window, sinks, ldo, out_scale, softcap,
+                                           gate, ldg}, st);
   if (direct) return;
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_gqa_merge<T>, dim3(d.Ttot, H), dim3(64), 0, st, pm, pl, pu, (T*)out, H, dv,
-                                          nsplit, sink, sink_logit, sinks, ldo, out_scale));
+                                          nsplit, sink, sink_logit, sinks, ldo, out_scale, (const T*)gate, ldg));
   LIPA_CHECK_LAUNCH();
 }
 

@@ -3,7 +3,7 @@
 // rows (no sort, no host round trip: decode steps and hipGraphs); and the weighted combine of expert outputs.
 // Routing variants (`kind` bits): scores as each output's own sigmoid instead of the softmax (1), a group ranked by the
 // sum of its two largest choices instead of its largest (2), weights divided by their sum over the chosen (4).
-// Experts are clipped GLUs or SiLU GLUs; the shared expert may sit behind a per-token sigmoid gate.
+// Experts are clipped GLUs or SiLU GLUs; a pair's weight multiplies the expert's output or its input; the shared expert may sit behind a per-token sigmoid gate.
 // Router scores, weights and the combine are float; expert products read the activation type and accumulate in float.
 #include "seq_common.h"
 
@@ -272,21 +272,24 @@ __device__ __forceinline__ float wave_dot<bf16>(const bf16* __restrict__ a, cons
 
 // pairs path, stage 1.  One wave per (pair, hidden unit r): a[pair, r] = glu(Wg_e[r] . h_t, Wu_e[r] . h_t).
 // wgu: [E, 2, F, W] (gate rows then up rows of every expert).  Identity pairs (e >= E) have nothing to compute.
+// inw (or null): a weight per pair that multiplies the expert's input, applied to both float products.
 template <typename T>
 __global__ __launch_bounds__(256) void k_moe_pair_up(const T* __restrict__ h, int ldh, const T* __restrict__ wgu,
                                                      const int* __restrict__ idx, T* __restrict__ a, int npairs, int top,
-                                                     int E, int F, int W, float limit, int mode) {
+                                                     int E, int F, int W, float limit, int mode,
+                                                     const float* __restrict__ inw) {
   const int pair = blockIdx.x, r = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int e = idx[pair];
   if (r >= F || e < 0 || e >= E) return;
   const T* x = h + (size_t)(pair / top) * ldh;
   const T* wg = wgu + ((size_t)e * 2 * F + r) * W;
-  const float g = wave_dot<T>(wg, x, W, lane), u = wave_dot<T>(wg + (size_t)F * W, x, W, lane);
+  const float iw = inw != nullptr ? inw[pair] : 1.f;
+  const float g = iw * wave_dot<T>(wg, x, W, lane), u = iw * wave_dot<T>(wg + (size_t)F * W, x, W, lane);
   if (lane == 0) a[(size_t)pair * F + r] = (T)glu(g, u, limit, mode);
 }
 
 // pairs path, stage 2.  One wave per (token, output column c):
-// out[t, c] = sum_j w[t, j] * (e_j < E ? Wd_e[c] . a[t, j] : h[t, c]) + shared[t, c]
+// out[t, c] = sum_j w[t, j] * (e_j < E ? Wd_e[c] . a[t, j] : h[t, c]) + shared[t, c]   (wts null: w = 1)
 template <typename T>
 __global__ __launch_bounds__(256) void k_moe_pair_down(const T* __restrict__ a, const T* __restrict__ wd,
                                                        const int* __restrict__ idx, const float* __restrict__ wts,
@@ -298,7 +301,7 @@ __global__ __launch_bounds__(256) void k_moe_pair_down(const T* __restrict__ a, 
   float acc = shared != nullptr ? (float)shared[(size_t)t * W + c] * (sgate != nullptr ? sigmoidf_(sgate[t]) : 1.f) : 0.f;
   for (int j = 0; j < top; ++j) {
     const int e = idx[(size_t)t * top + j];
-    const float w = wts[(size_t)t * top + j];
+    const float w = wts != nullptr ? wts[(size_t)t * top + j] : 1.f;
     if (e >= E)
       acc += w * (float)h[(size_t)t * ldh + c];
     else if (e >= 0)
@@ -331,7 +334,7 @@ __global__ __launch_bounds__(256) void k_moe_combine(const T* __restrict__ ys, c
 // mode 3 tanh-form GELU GLU of the [gate | up] halves of z [T, 2F]
 template <typename T>
 __global__ __launch_bounds__(256) void k_ff_act(const T* __restrict__ z, T* __restrict__ out, size_t n, int F, int mode,
-                                                float limit) {
+                                                float limit, const float* __restrict__ rs) {
   const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= n) return;
   if (mode == 0) {
@@ -339,7 +342,8 @@ __global__ __launch_bounds__(256) void k_ff_act(const T* __restrict__ z, T* __re
     out[i] = (T)gelu_tanhf_(v);
   } else {
     const size_t t = i / F, c = i % F;
-    out[i] = (T)glu((float)z[t * 2 * F + c], (float)z[t * 2 * F + F + c], limit, mode);
+    const float s = rs != nullptr ? rs[t] : 1.f;      // a weight per row on both halves
+    out[i] = (T)glu(s * (float)z[t * 2 * F + c], s * (float)z[t * 2 * F + F + c], limit, mode);
   }
 }
 
@@ -370,12 +374,13 @@ void seq_route_fused(int code, const void* h, int ldh, const float* router, cons
 
 void seq_moe_pairs(int code, const void* h, int ldh, const void* wgu, const void* wd, const int* idx, const float* wts,
                    const void* shared, const float* sgate, void* a, float* out, int T_, int top, int E, int F, int W,
-                   float limit, int mode, hipStream_t st) {
+                   float limit, int mode, int weight_input, hipStream_t st) {
   if (T_ == 0) return;
   SEQ_DISPATCH_T(code, {
     hipLaunchKernelGGL(k_moe_pair_up<T>, dim3(T_ * top, (F + 3) / 4), dim3(256), 0, st, (const T*)h, ldh, (const T*)wgu,
-                       idx, (T*)a, T_ * top, top, E, F, W, limit, mode);
-    hipLaunchKernelGGL(k_moe_pair_down<T>, dim3(T_, (W + 3) / 4), dim3(256), 0, st, (const T*)a, (const T*)wd, idx, wts,
+                       idx, (T*)a, T_ * top, top, E, F, W, limit, mode, weight_input ? wts : nullptr);
+    hipLaunchKernelGGL(k_moe_pair_down<T>, dim3(T_, (W + 3) / 4), dim3(256), 0, st, (const T*)a, (const T*)wd, idx,
+                       weight_input ? nullptr : wts,
                        (const T*)h, ldh, (const T*)shared, sgate, out, top, E, F, W);
   });
   LIPA_CHECK_LAUNCH();
@@ -389,10 +394,11 @@ void seq_moe_combine(int code, const void* ys, const long* pos, const int* idx, 
   LIPA_CHECK_LAUNCH();
 }
 
-void seq_ff_act(int code, const void* z, void* out, int T_, int F, int mode, float limit, hipStream_t st) {
+void seq_ff_act(int code, const void* z, void* out, int T_, int F, int mode, float limit, const float* row_scale,
+                hipStream_t st) {
   const size_t n = (size_t)T_ * F;
   if (n == 0) return;
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_ff_act<T>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, (const T*)z,
-                                          (T*)out, n, F, mode, limit));
+                                          (T*)out, n, F, mode, limit, row_scale));
   LIPA_CHECK_LAUNCH();
 }

@@ -101,14 +101,15 @@ __global__ __launch_bounds__(256) void k_polynorm(const T* __restrict__ z, const
   }
 }
 
-// out[t, h, c] = o[t, h, c] / rms_c(o[t, h, :]) * w[(per_head ? h * dv : 0) + c] * sigmoid(gate[t, h * dv + c]);
+// out[t, h, c] = o[t, h, c] / rms_c(o[t, h, :]) * w[(per_head ? h * dv : 0) + c] * sigmoid(gate[t, h * dv + c])
+// (times the gate itself with silu);
 // with den / efl (per token and head) o is first divided by max(|den|, efl) + 1e-6 (the mLSTM read-out)
 template <typename T>
 __global__ __launch_bounds__(256) void k_head_norm_gate(const float* __restrict__ o, const float* __restrict__ w,
                                                         int per_head, const T* __restrict__ gate, int ldg,
                                                         const float* __restrict__ den, const float* __restrict__ efl,
                                                         T* __restrict__ out, int ldo, float scale, int nrows, int H,
-                                                        int dv, float eps) {
+                                                        int dv, float eps, int silu) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (row >= nrows) return;
   const int t = row / H, hd = row % H;
@@ -121,7 +122,8 @@ __global__ __launch_bounds__(256) void k_head_norm_gate(const float* __restrict_
   }
   const float rs = rsqrtf(wave_sum(s) / dv + eps) * dinv;
   for (int c = lane; c < dv; c += 64) {
-    const float g = sigmoidf_((float)gate[(size_t)t * ldg + hd * dv + c]) * scale;
+    const float gp = (float)gate[(size_t)t * ldg + hd * dv + c];
+    const float g = sigmoidf_(gp) * (silu ? gp : 1.f) * scale;
     out[(size_t)t * ldo + hd * dv + c] = (T)(src[c] * rs * w[(per_head ? hd * dv : 0) + c] * g);
   }
 }
@@ -161,7 +163,7 @@ __global__ __launch_bounds__(256) void k_embed_pair(const long* __restrict__ tok
     float v = (float)table[(size_t)id * W + c] * scale;
     if (pair != nullptr) v += (float)pair[(size_t)row * W + c];
     x[(size_t)t * W + c] = v;
-    h[(size_t)t * W + c] = (T)v;
+    if (h != nullptr) h[(size_t)t * W + c] = (T)v;
   }
 }
 
@@ -468,28 +470,44 @@ __global__ __launch_bounds__(256) void k_qk_norm_store(const T* __restrict__ u, 
 
 // A step's [q | k (| v)] rows on their way into rotary attention: the first `dims` entries of every q and k head are
 // rotated at the token's position; the rotated k goes to the key cache; the value cache gets the v columns or, with
-// vkeys, the k columns as they came (a design whose values are its unrotated keys).  One block per token.
+// vkeys, the k columns as they came (a design whose values are its unrotated keys).  tevery > 0: q is multiplied by
+// 1 + tcoef ln(floor((pos + 1) / tevery) + 1).  veps >= 0: every head's value (dv entries) is divided by its root mean
+// square.  One block per token.
 template <typename T>
 __global__ __launch_bounds__(256) void k_rope_kv_store(const T* __restrict__ u, int ldu, const float* __restrict__ inv_freq,
                                                        T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
                                                        int nq, int nk, int nv, int dk, int dims, int half, float mag,
-                                                       int vkeys, int max_len, SeqDesc d) {
+                                                       int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
+                                                       SeqDesc d) {
   const size_t t = blockIdx.x;
   const T* r = u + t * ldu;
   const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]];
   const float p = (float)pos;
+  const float temp = tevery > 0 && pos >= 0 ? 1.f + tcoef * logf((float)((pos + 1) / tevery + 1)) : 1.f;
   for (int c = threadIdx.x; c < nq; c += 256) {
     const int cl = c % dk;
-    qout[t * nq + c] = (T)rotated_at(r + (c - cl), cl, dims, p, inv_freq, half, mag);
+    qout[t * nq + c] = (T)(rotated_at(r + (c - cl), cl, dims, p, inv_freq, half, mag) * temp);
   }
   if (pos < 0 || pos >= max_len) return;             // a row nobody reads may carry any position
   const size_t row = (size_t)slot * max_len + pos;
   for (int c = threadIdx.x; c < nk; c += 256) {
     const int cl = c % dk;
     kc[row * nk + c] = (T)rotated_at(r + nq + (c - cl), cl, dims, p, inv_freq, half, mag);
-    if (vkeys) vc[row * nk + c] = r[nq + c];
+    if (vkeys && veps < 0.f) vc[row * nk + c] = r[nq + c];
   }
-  if (!vkeys)
+  if (veps >= 0.f) {                                 // one wave per head: the value over its root mean square
+    const T* vr = r + (vkeys ? nq : nq + nk);
+    const int lane = threadIdx.x & 63;
+    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
+      float ss = 0.f;
+      for (int c = lane; c < dv; c += 64) {
+        const float v = (float)vr[h0 + c];
+        ss += v * v;
+      }
+      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
+      for (int c = lane; c < dv; c += 64) vc[row * nv + h0 + c] = (T)((float)vr[h0 + c] * rs);
+    }
+  } else if (!vkeys)
     for (int c = threadIdx.x; c < nv; c += 256) vc[row * nv + c] = r[nq + nk + c];
 }
 
@@ -577,11 +595,12 @@ __global__ __launch_bounds__(256) void k_delta_gates(const T* __restrict__ k, in
 }
 
 void seq_rope_kv_store(int code, const void* u, int ldu, const float* inv_freq, void* qout, void* kc, void* vc, int nq,
-                       int nk, int nv, int dk, int dims, int half, float mag, int vkeys, int max_len, SeqDesc d,
-                       hipStream_t st) {
+                       int nk, int nv, int dk, int dims, int half, float mag, int vkeys, int max_len, float tcoef,
+                       int tevery, float veps, int dv, SeqDesc d, hipStream_t st) {
   if (d.Ttot == 0) return;
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_rope_kv_store<T>, dim3(d.Ttot), dim3(256), 0, st, (const T*)u, ldu, inv_freq,
-                                          (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, d));
+                                          (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef,
+                                          tevery, veps, dv, d));
   LIPA_CHECK_LAUNCH();
 }
 
@@ -654,11 +673,11 @@ void seq_polynorm(int code, const void* z, const float* coef, void* out, int T_,
 
 void seq_head_norm_gate(int code, const float* o, const float* w, int per_head, const void* gate, int ldg,
                         const float* den, const float* efl, void* out, int ldo, float scale, int T_, int H, int dv,
-                        float eps, hipStream_t st) {
+                        float eps, int silu, hipStream_t st) {
   const int rows = T_ * H;
   if (rows == 0) return;
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_head_norm_gate<T>, dim3((rows + 3) / 4), dim3(256), 0, st, o, w, per_head,
-                                          (const T*)gate, ldg, den, efl, (T*)out, ldo, scale, rows, H, dv, eps));
+                                          (const T*)gate, ldg, den, efl, (T*)out, ldo, scale, rows, H, dv, eps, silu));
   LIPA_CHECK_LAUNCH();
 }
 

@@ -27,7 +27,7 @@ void seq_gated_residual(int, float*, const void*, int, const void*, int, const f
 void seq_dual_norm_mean(int, const void*, const void*, const float*, const float*, void*, int, int, float, hipStream_t);
 void seq_polynorm(int, const void*, const float*, void*, int, int, float, hipStream_t);
 void seq_head_norm_gate(int, const float*, const float*, int, const void*, int, const float*, const float*, void*, int,
-                        float, int, int, int, float, hipStream_t);
+                        float, int, int, int, float, int, hipStream_t);
 void seq_decay_gate(const float*, const float*, const float*, float*, int, int, int, hipStream_t);
 void seq_short_conv(int, int, const void*, int, const float*, const float*, void*, void*, int, int, int, const int*,
                     const float* const*, const float*, SeqDesc, float, hipStream_t);
@@ -50,7 +50,7 @@ void seq_route_grouped(const float*, const float*, int*, float*, int, int, int, 
 void seq_route_fused(int, const void*, int, const float*, const float*, int*, float*, int, int, int, int, int, int, float,
                      int, int, float*, hipStream_t);
 void seq_moe_pairs(int, const void*, int, const void*, const void*, const int*, const float*, const void*, const float*,
-                   void*, float*, int, int, int, int, int, float, int, hipStream_t);
+                   void*, float*, int, int, int, int, int, float, int, int, hipStream_t);
 void seq_moe_combine(int, const void*, const long*, const int*, const float*, const void*, int, const void*, const float*,
                      float*, int, int, int, int, hipStream_t);
 void seq_embed_learned(int, const long*, const int*, const void*, const void*, float*, int, int, int, int, int,
@@ -60,10 +60,21 @@ void seq_hyper_mix_norm(int, int, float*, const void*, int, const float*, const 
 void seq_qk_norm_store(int, const void*, int, const float*, const float*, void*, void*, void*, const void*, const float*,
                        int, int, int, int, float, SeqDesc, hipStream_t);
 void seq_gqa_attention(int, const void*, int, const void*, int, const void*, int, float*, float*, float*, const float*,
-                       int, int, int, int, float, const float*, void*, int, float, int, int, int, int, int, int, float,
-                       const int*, const int*, int, SeqDesc, hipStream_t);
+                       int, int, int, int, float, const float*, void*, int, float, float, const void*, int, int, int, int,
+                       int, int, int, float, const int*, const int*, int, SeqDesc, hipStream_t);
 void seq_rope_kv_store(int, const void*, int, const float*, void*, void*, void*, int, int, int, int, int, int, float, int,
-                       int, SeqDesc, hipStream_t);
+                       int, float, int, float, int, SeqDesc, hipStream_t);
+void seq_residual_dyt(int, int, const float*, const void*, int, float, float*, int, const float*, float*, const float*,
+                      const float*, float, const float*, int, const float*, float*, void*, int, const int*, const int*, int,
+                      SeqDesc, hipStream_t);
+void seq_softcap(float*, size_t, float, hipStream_t);
+void seq_selective_scan(int, const void*, int, const float*, const float*, const void*, int, const void*, int, const float*,
+                        const float*, const void*, int, float*, void*, int, float, int, int, SeqDesc, hipStream_t);
+void seq_gla_scan(int, const void*, int, const void*, int, const void*, int, const float*, const float*, float, float,
+                  float*, float*, int, int, int, SeqDesc, hipStream_t);
+int seq_dyt_max_taps();
+int seq_selective_max_states();
+int seq_gla_max_dk();
 void seq_sigmoid_gate(int, const void*, const void*, int, void*, int, int, hipStream_t);
 void seq_delta_gates(int, int, const void*, int, const void*, int, const float*, int, const float*, const void*, int,
                      const float*, float*, float*, float*, int, int, int, float, hipStream_t);
@@ -71,7 +82,7 @@ void seq_gdr_scan(int, const void*, int, const void*, int, const void*, int, con
                   float*, float*, int, int, int, SeqDesc, hipStream_t);
 int seq_hyper_max_streams();
 bool seq_attn_mfma_ok(int, int, int, int);
-void seq_ff_act(int, const void*, void*, int, int, int, float, hipStream_t);
+void seq_ff_act(int, const void*, void*, int, int, int, float, const float*, hipStream_t);
 int seq_route_max_outputs();
 void seq_mlstm_scan(int, const void*, int, const void*, int, const void*, int, const float*, const float*, const float*,
                     const float*, float, float, float*, float*, float*, float*, float*, float*, int, int, int, SeqDesc,
@@ -195,7 +206,7 @@ Tensor polynorm(Tensor z, Tensor coef, double eps) {
 
 // den / efl (optional, float [T, H]): o is divided by max(|den|, efl) + 1e-6 first
 Tensor head_norm_gate(Tensor o, Tensor w, Tensor gate, double eps, optional<Tensor> den, optional<Tensor> efl,
-                      optional<Tensor> out_, double scale) {
+                      optional<Tensor> out_, double scale, bool silu) {
   f32c(o, "o");
   TORCH_CHECK(o.dim() == 3, "o: [T, H, dv]");
   const int T = (int)o.size(0), H = (int)o.size(1), dv = (int)o.size(2), code = code_of(gate);
@@ -220,7 +231,7 @@ Tensor head_norm_gate(Tensor o, Tensor w, Tensor gate, double eps, optional<Tens
     ep = efl->data_ptr<float>();
   }
   seq_head_norm_gate(code, o.data_ptr<float>(), w.data_ptr<float>(), w.numel() != dv, gate.data_ptr(), ld(gate), dp, ep,
-                     out.data_ptr(), T == 0 ? H * dv : ld(out), (float)scale, T, H, dv, (float)eps, stream());
+                     out.data_ptr(), T == 0 ? H * dv : ld(out), (float)scale, T, H, dv, (float)eps, silu ? 1 : 0, stream());
   return out;
 }
 
@@ -423,7 +434,8 @@ Tensor ssd_scan(Tensor q, Tensor k, Tensor v, Tensor dtraw, Tensor dt_bias, Tens
 // returns {x float [T, W], h activation copy}; prev [slots] int32 (the token before a continued step), pair table
 // [buckets + 1, W] or none
 std::vector<Tensor> embed_pair(Tensor tok, Tensor table, optional<Tensor> pair, optional<Tensor> prev, double scale,
-                               int64_t mul_prev, int64_t mul_cur, std::vector<Tensor> desc, optional<Tensor> live) {
+                               int64_t mul_prev, int64_t mul_cur, std::vector<Tensor> desc, optional<Tensor> live,
+                               optional<Tensor> out_) {
   TORCH_CHECK(tok.is_cuda() && tok.scalar_type() == at::kLong && tok.is_contiguous(), "tokens: int64");
   TORCH_CHECK(table.is_cuda() && table.is_contiguous() && table.dim() == 2, "table");
   const int code = code_of(table);
@@ -442,10 +454,18 @@ std::vector<Tensor> embed_pair(Tensor tok, Tensor table, optional<Tensor> pair, 
     sp = prev->data_ptr<int>();
     buckets = pair->size(0) - 1;
   }
-  auto x = at::empty({T, W}, table.options().dtype(at::kFloat));
-  auto h = at::empty({T, W}, table.options());
-  seq_embed_pair(code, tok.data_ptr<long>(), table.data_ptr(), pp, sp, x.data_ptr<float>(), h.data_ptr(), (int)W,
-                 (float)scale, buckets, (long)mul_prev, (long)mul_cur, d, stream());
+  Tensor x, h;
+  if (out_ && out_->defined()) {                     // the float stream only, where the caller keeps it
+    x = *out_;
+    f32c(x, "out");
+    TORCH_CHECK(x.dim() == 2 && x.size(0) == T && x.size(1) == W, "out: [T, W]");
+  } else {
+    x = at::empty({T, W}, table.options().dtype(at::kFloat));
+    h = at::empty({T, W}, table.options());
+  }
+  seq_embed_pair(code, tok.data_ptr<long>(), table.data_ptr(), pp, sp, x.data_ptr<float>(),
+                 h.defined() ? h.data_ptr() : nullptr, (int)W, (float)scale, buckets, (long)mul_prev, (long)mul_cur, d,
+                 stream());
   return {x, h};
 }
 
@@ -574,7 +594,8 @@ Tensor latent_attention(Tensor qa, Tensor q, Tensor cache, optional<Tensor> gate
     auto pm = at::empty({np, H, nsplit}, fo), pl = at::empty({np, H, nsplit}, fo), pu = at::empty({np, H, nsplit, R}, fo);
     seq_gqa_attention(code, Q.data_ptr(), (int)(H * (R + dr)), cache.data_ptr(), (int)(R + dr), cache.data_ptr(),
                       (int)(R + dr), pm.data_ptr<float>(), pl.data_ptr<float>(), pu.data_ptr<float>(), nullptr, 0, 0,
-                      (int)window, has_sinks ? 1 : 0, 0.f, sp, out.data_ptr(), (int)(H * R), 1.f, (int)H, 1, (int)(R + dr),
+                      (int)window, has_sinks ? 1 : 0, 0.f, sp, out.data_ptr(), (int)(H * R), 1.f, 0.f, nullptr, 0, (int)H, 1,
+                      (int)(R + dr),
                       (int)R, (int)cache.size(1), (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
     return out;
   }
@@ -654,7 +675,7 @@ static const float* shared_gate_of(const optional<Tensor>& sg, int64_t T) {
 }
 
 Tensor moe_pairs(Tensor h, Tensor wgu, Tensor wd, Tensor idx, Tensor w, optional<Tensor> shared, double limit,
-                 int64_t mode, optional<Tensor> shared_gate) {
+                 int64_t mode, optional<Tensor> shared_gate, bool weight_input) {
   TORCH_CHECK(mode == 1 || mode == 2, "expert activation: 1 clipped GLU, 2 SiLU GLU");
   const int code = code_of(h);
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.is_contiguous(), "h: [T, W] contiguous");
@@ -677,7 +698,7 @@ Tensor moe_pairs(Tensor h, Tensor wgu, Tensor wd, Tensor idx, Tensor w, optional
   auto out = at::empty({T, W}, h.options().dtype(at::kFloat));
   seq_moe_pairs(code, h.data_ptr(), (int)W, wgu.data_ptr(), wd.data_ptr(), idx.data_ptr<int>(), w.data_ptr<float>(), sp,
                 shared_gate_of(shared_gate, T), a.data_ptr(), out.data_ptr<float>(), (int)T, (int)top, (int)E, (int)F,
-                (int)W, (float)limit, (int)mode, stream());
+                (int)W, (float)limit, (int)mode, weight_input ? 1 : 0, stream());
   return out;
 }
 
@@ -706,12 +727,19 @@ Tensor moe_combine_sorted(Tensor ys, Tensor pos, Tensor idx, Tensor w, Tensor h,
 
 // mode 0: tanh-form GELU of z [T, F]; mode 1: clipped GLU, mode 2: SiLU GLU, mode 3: tanh-form GELU GLU of
 // z [T, 2F] = [gate | up]
-Tensor ff_act(Tensor z, int64_t mode, double limit) {
+// row_scale (float [T] or none): both halves of a GLU's row are multiplied by it first
+Tensor ff_act(Tensor z, int64_t mode, double limit, optional<Tensor> row_scale) {
   TORCH_CHECK(z.is_cuda() && z.is_contiguous() && z.dim() == 2 &&
                   (mode == 0 || (mode >= 1 && mode <= 3 && z.size(1) % 2 == 0)), "z");
   const int64_t T = z.size(0), F = mode == 0 ? z.size(1) : z.size(1) / 2;
   auto out = at::empty({T, F}, z.options());
-  seq_ff_act(code_of(z), z.data_ptr(), out.data_ptr(), (int)T, (int)F, (int)mode, (float)limit, stream());
+  const float* rp = nullptr;
+  if (row_scale && row_scale->defined()) {
+    f32c(*row_scale, "row_scale");
+    TORCH_CHECK(mode != 0 && row_scale->numel() == T, "row_scale: [T], with a GLU");
+    rp = row_scale->data_ptr<float>();
+  }
+  seq_ff_act(code_of(z), z.data_ptr(), out.data_ptr(), (int)T, (int)F, (int)mode, (float)limit, rp, stream());
   return out;
 }
 
@@ -804,7 +832,7 @@ Tensor qk_norm_store(Tensor u, int64_t nq, int64_t nk, Tensor qw, Tensor kw, Ten
 Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, int64_t H, int64_t G, double scale,
                         int64_t block, bool sink, double sink_logit, int64_t nsplit, std::vector<Tensor> desc,
                         std::vector<Tensor> tiles, int64_t window, optional<Tensor> sinks, optional<Tensor> out_,
-                        double out_scale) {
+                        double out_scale, double softcap, optional<Tensor> gate) {
   const int code = code_of(q);
   TORCH_CHECK(q.dim() == 2 && H >= 1 && G >= 1 && H % G == 0 && q.size(1) % H == 0, "q: [T, H * dk]");
   const int64_t T = q.size(0), dk = q.size(1) / H;
@@ -851,6 +879,15 @@ Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, i
   }
   const int ldo = T == 0 ? (int)(H * dv) : ld(out);
   if (ldo % 4 != 0 || ((uintptr_t)out.data_ptr() & 7) != 0) tseq = nullptr;    // the matrix-core sweep stores 8 bytes
+  TORCH_CHECK(softcap >= 0, "softcap");
+  const void* gp = nullptr;
+  int ldg = 0;
+  if (gate && gate->defined()) {
+    rows(*gate, T, H * dv, code, "gate");
+    gp = gate->data_ptr();
+    ldg = T == 0 ? (int)(H * dv) : ld(*gate);
+    if (ldg % 4 != 0 || ((uintptr_t)gp & 7) != 0) tseq = nullptr;              // and reads the gate 8 bytes at a time
+  }
   // one key split on the matrix-core sweep writes the output itself: no partial sums
   const bool direct = nsplit == 1 && tseq != nullptr && seq_attn_mfma_ok(code, ld(q), (int)dk, (int)dv) &&
                       (G * dk) % 8 == 0 && (G * dv) % 8 == 0;
@@ -859,20 +896,22 @@ Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, i
   auto pu = at::empty({np, H, nsplit, dv}, fo);
   seq_gqa_attention(code, q.data_ptr(), ld(q), kc.data_ptr(), (int)(G * dk), vc.data_ptr(), (int)(G * dv),
                     pm.data_ptr<float>(), pl.data_ptr<float>(), pu.data_ptr<float>(), bp, nd, (int)block, (int)window,
-                    sink ? 1 : 0, (float)sink_logit, sp, out.data_ptr(), ldo, (float)out_scale, (int)H, (int)G, (int)dk,
-                    (int)dv, (int)max_len, (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
+                    sink ? 1 : 0, (float)sink_logit, sp, out.data_ptr(), ldo, (float)out_scale, (float)softcap, gp, ldg, (int)H,
+                    (int)G, (int)dk, (int)dv, (int)max_len, (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
   return out;
 }
 
 // u [T, nq + nk (+ nv)]: rotated q returned, rotated k and the values (u's v columns, or the k columns as they came) go
 // to the caches at each token's (slot, position)
 Tensor rope_kv_store(Tensor u, int64_t nq, int64_t nk, int64_t H, int64_t G, Tensor inv_freq, int64_t dims, Tensor kc,
-                     Tensor vc, std::vector<Tensor> desc, bool half, double mag, bool values_are_keys) {
+                     Tensor vc, std::vector<Tensor> desc, bool half, double mag, bool values_are_keys, double temp_coef,
+                     int64_t temp_every, double v_eps) {
   const int code = code_of(u);
   TORCH_CHECK(u.dim() == 2 && H >= 1 && G >= 1 && nq % H == 0 && nk % G == 0 && nq / H == nk / G &&
                   u.size(1) >= nq + nk, "u: [T, H * dk + G * dk (+ nv)]");
   const int64_t T = u.size(0), nv = values_are_keys ? nk : u.size(1) - nq - nk, dk = nq / H;
-  TORCH_CHECK(nv >= 1, "no value columns");
+  TORCH_CHECK(nv >= 1 && nv % G == 0, "value columns: G * dv");
+  TORCH_CHECK(temp_every >= 0 && temp_every < (1ll << 31), "query temperature");
   rows(u, T, u.size(1), code, "u");
   check_freq(inv_freq, dims, dk);
   check_kv_cache(kc, nk, code, "key cache");
@@ -882,8 +921,146 @@ Tensor rope_kv_store(Tensor u, int64_t nq, int64_t nk, int64_t H, int64_t G, Ten
   auto q = at::empty({T, nq}, u.options());
   seq_rope_kv_store(code, u.data_ptr(), ld(u), inv_freq.data_ptr<float>(), q.data_ptr(), kc.data_ptr(), vc.data_ptr(),
                     (int)nq, (int)nk, (int)nv, (int)dk, (int)dims, half ? 1 : 0, (float)mag, values_are_keys ? 1 : 0,
-                    (int)kc.size(1), d, stream());
+                    (int)kc.size(1), (float)temp_coef, (int)temp_every, (float)v_eps, (int)(nv / G), d, stream());
   return q;
+}
+
+// x [T, W] float (not written), y none / float / the activation dtype; streams [L + 1, T, W], depth [n + 1] or none;
+// conv [taps, W] or none with state [slots, taps - 1, W] (written) and old (read: the state itself, or a copy of it when
+// several blocks share a continued sequence).  Returns {r, h}.
+std::vector<Tensor> residual_dyt(Tensor x, optional<Tensor> y, double mult, Tensor w, Tensor b, double alpha, bool out_bf16,
+                                 optional<Tensor> conv, optional<Tensor> state, optional<Tensor> old,
+                                 optional<Tensor> streams, int64_t n, optional<Tensor> depth, std::vector<Tensor> desc,
+                                 optional<Tensor> live, std::vector<Tensor> tiles) {
+  f32c(x, "x");
+  TORCH_CHECK(x.dim() == 2, "x: [T, W]");
+  const int64_t T = x.size(0), W = x.size(1);
+  const int code = out_bf16 ? 0 : 1;
+  f32c(w, "norm weight");
+  f32c(b, "norm bias");
+  TORCH_CHECK(w.numel() == W && b.numel() == W, "norm weight and bias: [W]");
+  const void* yp = nullptr;
+  int y_f32 = 0, ldy = 0;
+  if (y && y->defined()) {
+    y_f32 = y->scalar_type() == at::kFloat;
+    rows(*y, T, W, code_of(*y), "y");
+    TORCH_CHECK(y_f32 || code_of(*y) == code, "y: float or the activation dtype");
+    yp = y->data_ptr();
+    ldy = T == 0 ? (int)W : ld(*y);
+  }
+  float* sp = nullptr;
+  const float* dp = nullptr;
+  if (depth && depth->defined()) {
+    f32c(*depth, "depth weights");
+    TORCH_CHECK(streams && streams->defined(), "a depth average needs the streams");
+    f32c(*streams, "streams");
+    TORCH_CHECK(streams->dim() == 3 && streams->size(1) == T && streams->size(2) == W && n >= 0 && n < streams->size(0) &&
+                    depth->numel() == n + 1, "streams: [layers + 1, T, W], depth weights: [n + 1]");
+    sp = streams->data_ptr<float>();
+    dp = depth->data_ptr<float>();
+    TORCH_CHECK(T == 0 || x.data_ptr<float>() != sp + (size_t)n * T * W, "x must not be the stream that is written");
+  }
+  SeqDesc d{nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, (int)T};
+  const float* cp = nullptr;
+  const float* sin = nullptr;
+  float* sout = nullptr;
+  const int *tseq = nullptr, *tt0 = nullptr;
+  int taps = 0, ntiles = 0;
+  if (conv && conv->defined()) {
+    f32c(*conv, "convolution");
+    TORCH_CHECK(conv->dim() == 2 && conv->size(1) == W && conv->size(0) >= 1 && conv->size(0) <= seq_dyt_max_taps(),
+                "convolution: [taps, W], at most ", seq_dyt_max_taps(), " taps");
+    taps = (int)conv->size(0);
+    cp = conv->data_ptr<float>();
+    d = desc_of(desc, live, T);
+    if (taps > 1) {
+      TORCH_CHECK(state && state->defined() && old && old->defined(), "a convolution carries rows");
+      f32c(*state, "carried rows");
+      f32c(*old, "carried rows");
+      TORCH_CHECK(state->dim() == 3 && state->size(1) == taps - 1 && state->size(2) == W && old->sizes() == state->sizes(),
+                  "carried rows: [slots, taps - 1, W]");
+      sin = old->data_ptr<float>();
+      sout = state->data_ptr<float>();
+    }
+    TORCH_CHECK(tiles.size() == 2 && tiles[0].numel() == tiles[1].numel(), "tiles: two arrays of one length");
+    for (auto& t : tiles) TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous(), "tiles: int32");
+    ntiles = (int)tiles[0].numel();
+    TORCH_CHECK((int64_t)ntiles * 32 >= T, "tiles must cover the tokens");
+    tseq = tiles[0].data_ptr<int>();
+    tt0 = tiles[1].data_ptr<int>();
+  }
+  const bool same = yp == nullptr && dp == nullptr;  // nothing was added: r is x
+  auto r = same ? x : at::empty({T, W}, x.options());
+  auto h = at::empty({T, W}, x.options().dtype(out_bf16 ? at::kBFloat16 : at::kFloat));
+  seq_residual_dyt(code, y_f32, x.data_ptr<float>(), yp, ldy, (float)mult, sp, (int)n, dp, same ? nullptr : r.data_ptr<float>(),
+                   w.data_ptr<float>(), b.data_ptr<float>(), (float)alpha, cp, taps, sin, sout, h.data_ptr(), (int)W, tseq, tt0,
+                   ntiles, d, stream());
+  return {r, h};
+}
+
+Tensor softcap_(Tensor z, double cap) {
+  f32c(z, "logits");
+  TORCH_CHECK(cap > 0, "softcap");
+  seq_softcap(z.data_ptr<float>(), (size_t)z.numel(), (float)cap, stream());
+  return z;
+}
+
+// x, z [T, C], b, c [T, N] activation rows, dt_pre float [T, C] contiguous; S float [slots, C, N] in place
+Tensor selective_scan(Tensor x, Tensor dt_pre, Tensor dt_bias, Tensor b, Tensor c, Tensor a_log, Tensor d_skip, Tensor z,
+                      Tensor S, std::vector<Tensor> desc, optional<Tensor> live, optional<Tensor> out_, double scale) {
+  const int code = code_of(x);
+  TORCH_CHECK(x.dim() == 2 && b.dim() == 2, "x: [T, C], b: [T, N]");
+  const int64_t T = x.size(0), C = x.size(1), N = b.size(1);
+  rows(x, T, C, code, "x");
+  rows(z, T, C, code, "z");
+  rows(b, T, N, code, "b");
+  rows(c, T, N, code, "c");
+  f32c(dt_pre, "dt_pre");
+  f32c(dt_bias, "dt_bias");
+  f32c(a_log, "A_log");
+  f32c(d_skip, "D");
+  TORCH_CHECK(dt_pre.numel() == T * C && dt_bias.numel() == C && d_skip.numel() == C && a_log.numel() == C * N,
+              "dt_pre [T, C], dt_bias and D [C], A_log [C, N]");
+  TORCH_CHECK(N >= 1 && N <= seq_selective_max_states(), "selective scan: 1..", seq_selective_max_states(), " states");
+  f32c(S, "state");
+  TORCH_CHECK(S.dim() == 3 && S.size(1) == C && S.size(2) == N, "state: [slots, C, N]");
+  SeqDesc d = desc_of(desc, live, T);
+  Tensor out;
+  if (out_ && out_->defined()) {                     // a column slice of a wider matrix
+    out = *out_;
+    rows(out, T, C, code, "out");
+  } else {
+    out = at::empty({T, C}, x.options());
+  }
+  if (T == 0) return out;
+  seq_selective_scan(code, x.data_ptr(), ld(x), dt_pre.data_ptr<float>(), dt_bias.data_ptr<float>(), b.data_ptr(), ld(b),
+                     c.data_ptr(), ld(c), a_log.data_ptr<float>(), d_skip.data_ptr<float>(), z.data_ptr(), ld(z),
+                     S.data_ptr<float>(), out.data_ptr(), ld(out), (float)scale, (int)C, (int)N, d, stream());
+  return out;
+}
+
+// q, k [T, H * dk], v [T, H * dv] activation rows, z float [T, H * dk] contiguous; S float [slots, H, dv, dk] in place
+Tensor gated_linear_scan(Tensor q, Tensor k, Tensor v, Tensor z, Tensor z_bias, double tau, double q_scale, Tensor S,
+                         int64_t H, std::vector<Tensor> desc, optional<Tensor> live) {
+  const int code = code_of(q);
+  TORCH_CHECK(H >= 1 && q.dim() == 2 && q.size(1) % H == 0 && v.dim() == 2 && v.size(1) % H == 0,
+              "q/k: [T, H * dk], v: [T, H * dv]");
+  const int64_t T = q.size(0), dk = q.size(1) / H, dv = v.size(1) / H;
+  rows(q, T, H * dk, code, "q");
+  rows(k, T, H * dk, code, "k");
+  rows(v, T, H * dv, code, "v");
+  f32c(z, "z");
+  f32c(z_bias, "z_bias");
+  TORCH_CHECK(z.numel() == T * H * dk && z_bias.numel() == H * dk && tau > 0, "z [T, H * dk], z_bias [H * dk], tau > 0");
+  TORCH_CHECK(dk >= 1 && dk <= seq_gla_max_dk() && dv >= 1, "gated linear attention: key size above ", seq_gla_max_dk());
+  check_state(S, H, dv, dk);
+  SeqDesc d = desc_of(desc, live, T);
+  auto out = at::empty({T, H, dv}, S.options());
+  if (T == 0) return out;
+  seq_gla_scan(code, q.data_ptr(), ld(q), k.data_ptr(), ld(k), v.data_ptr(), ld(v), z.data_ptr<float>(),
+               z_bias.data_ptr<float>(), (float)(1.0 / tau), (float)q_scale, S.data_ptr<float>(), out.data_ptr<float>(), (int)H,
+               (int)dk, (int)dv, d, stream());
+  return out;
 }
 
 Tensor sigmoid_gate(Tensor y, Tensor gate) {
@@ -977,7 +1154,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("delta_scan", &delta_scan);
   m.def("talk_attention", &talk_attention);
   m.def("ssd_scan", &ssd_scan);
-  m.def("embed_pair", &embed_pair);
+  m.def("embed_pair", &embed_pair, py::arg("tok"), py::arg("table"), py::arg("pair"), py::arg("prev"), py::arg("scale"),
+        py::arg("mul_prev"), py::arg("mul_cur"), py::arg("desc"), py::arg("live"), py::arg("out") = py::none());
   m.def("scaled_postnorm", &scaled_postnorm);
   m.def("rms_act", &rms_act);
   m.def("gate_group_norm", &gate_group_norm);
@@ -987,13 +1165,17 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route_fused", &route_fused);
   m.def("moe_pairs", &moe_pairs);
   m.def("moe_combine_sorted", &moe_combine_sorted);
-  m.def("ff_act", &ff_act);
+  m.def("ff_act", &ff_act, py::arg("z"), py::arg("mode"), py::arg("limit"), py::arg("row_scale") = py::none());
   m.def("embed_learned", &embed_learned);
   m.def("hyper_mix_norm", &hyper_mix_norm);
   m.def("qk_norm_store", &qk_norm_store);
   m.def("biased_attention", &biased_attention);
   m.def("rope_kv_store", &rope_kv_store);
   m.def("sigmoid_gate", &sigmoid_gate);
+  m.def("residual_dyt", &residual_dyt);
+  m.def("softcap_", &softcap_);
+  m.def("selective_scan", &selective_scan);
+  m.def("gated_linear_scan", &gated_linear_scan);
   m.def("delta_rule_gates", &delta_rule_gates);
   m.def("general_delta_scan", &general_delta_scan);
 }
