@@ -421,15 +421,28 @@ __global__ __launch_bounds__(64) void k_gqa_merge(const float* __restrict__ pm, 
   const int t = blockIdx.x, g = blockIdx.y, lane = threadIdx.x;
   const size_t b = ((size_t)t * H + g) * nsplit;
   if (sinks != nullptr) sink_logit = sinks[g];
+  // a lane takes split z = lane (+ 64 ...): maximum and denominator are wave reductions, a split's weight is handed round
   float mx = sink ? sink_logit : -INFINITY;
-  for (int z = 0; z < nsplit; ++z) mx = fmaxf(mx, pm[b + z]);
-  float l = sink ? expf(sink_logit - mx) : 0.f;
-  for (int z = 0; z < nsplit; ++z) l += pm[b + z] == -INFINITY ? 0.f : expf(pm[b + z] - mx) * pl[b + z];
+  for (int z = lane; z < nsplit; z += 64) mx = fmaxf(mx, pm[b + z]);
+  mx = wave_max(mx);
+  float l = 0.f;
+  for (int z = lane; z < nsplit; z += 64) l += pm[b + z] == -INFINITY ? 0.f : expf(pm[b + z] - mx) * pl[b + z];
+  l = wave_sum(l) + (sink ? expf(sink_logit - mx) : 0.f);
   const float inv = l > 0.f ? out_scale / l : 0.f;
-  for (int col = lane; col < dv; col += 64) {
+  for (int c0 = 0; c0 < dv; c0 += 64) {
+    const int col = c0 + lane;
     float u = 0.f;
-    for (int z = 0; z < nsplit; ++z)
-      if (pm[b + z] != -INFINITY) u += expf(pm[b + z] - mx) * pu[(b + z) * dv + col];
+    for (int z0 = 0; z0 < nsplit; z0 += 64) {
+      const int nz = min(64, nsplit - z0);
+      const float mz = lane < nz ? pm[b + z0 + lane] : -INFINITY;
+      const float wz = mz == -INFINITY ? 0.f : expf(mz - mx);
+#pragma unroll 8
+      for (int z = 0; z < nz; ++z) {
+        const float w = __shfl(wz, z, 64);            // (an empty split has weight 0; its sums were written as 0)
+        if (col < dv) u += w * pu[(b + z0 + z) * dv + col];
+      }
+    }
+    if (col >= dv) continue;
     if (gate != nullptr) u *= sigmoidf_((float)gate[(size_t)t * ldg + g * dv + col]);
     out[(size_t)t * ldo + g * dv + col] = (T)(u * inv);
   }

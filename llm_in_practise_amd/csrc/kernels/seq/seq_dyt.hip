@@ -62,7 +62,8 @@ struct DytArgs {
   const float* sin;      // [slots, taps - 1, W] carried rows, read
   float* sout;           // the same, written
   int W;
-  const int *tile_seq, *tile_t0;   // null: plain runs of RUN rows (no convolution)
+  const int *tile_seq, *tile_t0;
+  int run;               // tokens per block without a convolution
 };
 
 // r of token t, columns [c, c + V): x + mult y, then the average over depth (the streams before this one are read, this
@@ -114,7 +115,7 @@ __global__ __launch_bounds__(64) void k_residual_dyt(DytArgs a, const float* __r
     return o;
   };
   if constexpr (TP == 1) {
-    const int t0 = blockIdx.x * RUN, t1 = min(t0 + RUN, d.Ttot);
+    const int t0 = blockIdx.x * a.run, t1 = min(t0 + a.run, d.Ttot);
     for (int t = t0; t < t1; ++t) stv<V>(h + (size_t)t * a.W + c, normed(residual_at<YT, V, true>(a, x, y, streams, depth, sn, rout, t, c)));
   } else {
     const int tile = blockIdx.x >> 1, s = a.tile_seq[tile], s0 = d.seq_off[s], s1 = d.seq_off[s + 1];
@@ -176,7 +177,7 @@ void launch_dyt(const DytArgs& a, const float* x, const void* y, float* streams,
   float* sn = depth != nullptr ? streams + (size_t)a.n * a.sstride : nullptr;
   const int V = vec ? 4 : 1;
   const unsigned gy = (unsigned)((a.W + 64 * V - 1) / (64 * V));
-  const dim3 grid(a.conv != nullptr ? 2 * ntiles : (d.Ttot + RUN - 1) / RUN, gy);
+  const dim3 grid(a.conv != nullptr ? 2 * ntiles : (d.Ttot + a.run - 1) / a.run, gy);
 #define DYT_LAUNCH(V_, TP_) \
   hipLaunchKernelGGL((k_residual_dyt<T, YT, V_, TP_>), grid, dim3(64), 0, st, a, x, (const YT*)y, \
                      streams, depth, sn, r, (T*)h, d)
@@ -200,7 +201,8 @@ void seq_residual_dyt(int code, int y_f32, const float* x, const void* y, int ld
                       const float* sin, float* sout, void* h, int W, const int* tile_seq, const int* tile_t0, int ntiles,
                       SeqDesc d, hipStream_t st) {
   if (d.Ttot == 0) return;
-  const DytArgs a{ldy, mult, (size_t)d.Ttot * W, n, w, b, alpha, conv, taps, sin, sout, W, tile_seq, tile_t0};
+  const DytArgs a{ldy, mult, (size_t)d.Ttot * W, n, w, b, alpha, conv, taps, sin, sout, W, tile_seq, tile_t0,
+                  d.Ttot < 1024 ? 1 : RUN};
   const bool vec = W % 4 == 0 && (y == nullptr || (ldy % 4 == 0 && ((uintptr_t)y & 15) == 0));   // the rest: whole tensors
   SEQ_DISPATCH_T(code, {
     if (y_f32)

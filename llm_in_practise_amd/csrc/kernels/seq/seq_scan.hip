@@ -85,6 +85,74 @@ __global__ __launch_bounds__(64) void k_short_conv(const T* __restrict__ u, int 
   }
 }
 
+// The same for segments without a norm (plain or SiLU), four channels per thread: a wave owns 256 channels of a run of
+// consecutive packed tokens and keeps the last TP - 1 inputs in registers (TP: taps rounded up; missing taps weigh 0), so an
+// input is read once per run instead of once per tap.  At a sequence's first token of the run the window is read again
+// (from the step's tokens, the carried rows or as zeros).  `roll`: every sequence has exactly one token in this step; the
+// thread that read its carried rows writes them back shifted.
+__device__ __forceinline__ f32x4 conv_ld4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+__device__ __forceinline__ f32x4 conv_ld4(const bf16* p) {
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+__device__ __forceinline__ void conv_st4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+__device__ __forceinline__ void conv_st4(bf16* p, f32x4 v) {
+  *reinterpret_cast<bf16x4*>(p) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+}
+
+template <typename T, typename OT, int TP>
+__global__ __launch_bounds__(64) void k_conv_run(const T* __restrict__ u, int ldu, const float* __restrict__ w,
+                                                 const float* __restrict__ bias, T* __restrict__ state,
+                                                 OT* __restrict__ out, int C, int taps, int run, int roll, ConvArgs a,
+                                                 SeqDesc d) {
+  const int c = (blockIdx.y * 64 + threadIdx.x) * 4, t0 = blockIdx.x * run, t1 = min(t0 + run, d.Ttot), keep = taps - 1;
+  if (c >= C) return;
+  int si = 0;
+  while (si < a.nseg - 1 && c >= a.seg[si + 1].c0) ++si;
+  const bool silu = a.seg[si].mode == 2;
+  f32x4 cw[TP], win[TP - 1], b = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < TP; ++j)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) cw[j][i] = j >= TP - taps ? w[(size_t)(c + i) * taps + j - (TP - taps)] : 0.f;
+  if (bias != nullptr) b = conv_ld4(bias + c);
+  int cur = -1, slot = 0;
+  for (int t = t0; t < t1; ++t) {
+    const int s = d.tok_seq[t];
+    if (s != cur) {
+      cur = s;
+      slot = d.slots[s];
+      const int s0 = d.seq_off[s], p0 = d.pos0[s];
+#pragma unroll
+      for (int j = 0; j < TP - 1; ++j) {
+        const int li = t - s0 - (TP - 1) + j;
+        win[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (j >= TP - 1 - keep) {
+          if (li >= 0)
+            win[j] = conv_ld4(u + (size_t)(s0 + li) * ldu + c);
+          else if (p0 > 0)
+            win[j] = conv_ld4(state + ((size_t)slot * keep + keep + li) * C + c);
+        }
+      }
+    }
+    const f32x4 x = conv_ld4(u + (size_t)t * ldu + c);
+    f32x4 y = b + cw[TP - 1] * x;
+#pragma unroll
+    for (int j = 0; j < TP - 1; ++j) y += cw[j] * win[j];
+    if (silu)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) y[i] *= sigmoidf_(y[i]);
+    conv_st4(out + (size_t)t * C + c, y);
+#pragma unroll
+    for (int j = 0; j < TP - 2; ++j) win[j] = win[j + 1];
+    win[TP - 2] = x;
+    if (roll && !(d.live && !d.live[s]))
+#pragma unroll
+      for (int j = 0; j < TP - 1; ++j)
+        if (j >= TP - 1 - keep) conv_st4(state + ((size_t)slot * keep + j - (TP - 1 - keep)) * C + c, win[j]);
+  }
+}
+
 // the last taps-1 inputs of every sequence become its carried state (older ones shift out)
 template <typename T>
 __global__ __launch_bounds__(256) void k_conv_state(const T* __restrict__ u, int ldu, T* __restrict__ state, int C,
@@ -575,6 +643,28 @@ void seq_short_conv(int code, int out_f32, const void* u, int ldu, const float* 
   for (int i = 0; i < nseg; ++i) {
     a.seg[i] = ConvSeg{segs[4 * i], segs[4 * i + 1], segs[4 * i + 2], segs[4 * i + 3], sw[i], sscale[i]};
     heads += segs[4 * i + 1];
+  }
+  bool run4 = C % 4 == 0 && ldu % 4 == 0 && ((uintptr_t)u & 15) == 0;       // 16-byte rows, no norm in any segment
+  for (int i = 0; i < nseg; ++i) run4 = run4 && (a.seg[i].mode == 0 || a.seg[i].mode == 2) && a.seg[i].c0 % 4 == 0;
+  if (run4) {
+    const int run = d.Ttot < 1024 ? 1 : 16, roll = d.Ttot == d.B && taps > 1;
+    const dim3 grid((d.Ttot + run - 1) / run, (C + 255) / 256);
+#define CONV_RUN(OT, TP)                                                                                              \
+  hipLaunchKernelGGL((k_conv_run<T, OT, TP>), grid, dim3(64), 0, st, (const T*)u, ldu, w, bias, (T*)state, (OT*)out, C, \
+                     taps, run, roll, a, d)
+    SEQ_DISPATCH_T(code, {
+      if (taps <= 4) {
+        if (out_f32) CONV_RUN(float, 4); else CONV_RUN(T, 4);
+      } else {
+        if (out_f32) CONV_RUN(float, 8); else CONV_RUN(T, 8);
+      }
+      if (taps > 1 && !roll)
+        hipLaunchKernelGGL(k_conv_state<T>, dim3(d.B, (C + 255) / 256), dim3(256), 0, st, (const T*)u, ldu, (T*)state, C,
+                           taps, d);
+    });
+#undef CONV_RUN
+    LIPA_CHECK_LAUNCH();
+    return;
   }
   SEQ_DISPATCH_T(code, {
     if (out_f32)

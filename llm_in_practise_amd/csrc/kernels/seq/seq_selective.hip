@@ -12,10 +12,58 @@ namespace {
 
 constexpr int CT = 16;      // tokens staged per chunk
 
-template <int CTRL>
-__device__ __forceinline__ float dpp_add_(float v) {
-  return v + __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), CTRL, 0xF, 0xF, true));
+// ln(1 + e^-a) for a >= 0 as 2 atanh(e / (2 + e)), e = e^-a: the argument stays below 1/3, so eight terms of the odd series
+// reach float accuracy without a table or a branch (the staging of a chunk evaluates one per element).
+__device__ __forceinline__ float log1p_exp_neg(float a) {
+  const float e = __builtin_amdgcn_exp2f(a * -1.4426950408889634f), s = e * __builtin_amdgcn_rcpf(2.f + e), q = s * s;
+  float p = 1.f / 17.f;
+  p = p * q + 1.f / 15.f;
+  p = p * q + 1.f / 13.f;
+  p = p * q + 1.f / 11.f;
+  p = p * q + 1.f / 9.f;
+  p = p * q + 1.f / 7.f;
+  p = p * q + 1.f / 5.f;
+  p = p * q + 1.f / 3.f;
+  return 2.f * s * (p * q + 1.f);
 }
+__device__ __forceinline__ float softplus_fast(float x) { return fmaxf(x, 0.f) + log1p_exp_neg(fabsf(x)); }
+__device__ __forceinline__ float silu_fast(float z) {
+  return z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f));
+}
+
+// Lane layout of a wave: R lanes (4, 8 or 16) share a column; they differ in lane bits 4 and 5 (the wave's rows of 16
+// lanes) and, above four, in bits 0 and 1.  The other bits tell the wave's 64 / R column groups apart.
+template <int R>
+__device__ __forceinline__ int lane_part(int lane) {
+  return (lane >> 4) | (R >= 8 ? (lane & 1) << 2 : 0) | (R >= 16 ? (lane & 2) << 2 : 0);
+}
+template <int R>
+__device__ __forceinline__ int lane_group(int lane) {
+  return R == 4 ? lane & 15 : R == 8 ? (lane & 15) >> 1 : (lane & 15) >> 2;
+}
+// Four values summed over a column's R lanes at once: after exchanging halves of the wave and rows of 16 lanes, row i of
+// the wave holds value i (in all lanes of its group): two exchanges and an exchange of sums instead of four butterflies.
+__device__ __forceinline__ float dpp_quad_add(float v, int which) {
+  const int o = which == 0 ? __builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, true)     // quad_perm [1, 0, 3, 2]
+                           : __builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xF, 0xF, true);    // quad_perm [2, 3, 0, 1]
+  return v + __int_as_float(o);
+}
+__device__ __forceinline__ float swap32_add(float a, float b) {       // lanes 0-31: sum of a, lanes 32-63: sum of b
+  const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(a), __float_as_uint(b), false, false);
+  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+__device__ __forceinline__ float swap16_add(float a, float b) {       // even rows: sum of a over a pair of rows, odd: of b
+  const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(a), __float_as_uint(b), false, false);
+  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+template <int R>
+__device__ __forceinline__ float sum_four(float v0, float v1, float v2, float v3) {
+  float v = swap16_add(swap32_add(v0, v2), swap32_add(v1, v3));
+  if (R >= 8) v = dpp_quad_add(v, 0);
+  if (R >= 16) v = dpp_quad_add(v, 1);
+  return v;
+}
+
 // NR contiguous entries of a state row of `len`, starting at i0 (past the row's end: 0); 16-byte accesses where they fit
 template <int NR>
 __device__ __forceinline__ void load_state(const float* p, int i0, int len, bool on, float (&r)[NR]) {
@@ -49,23 +97,16 @@ __device__ __forceinline__ void store_state(float* p, int i0, int len, const flo
   }
 }
 
-// sum over R adjacent lanes (R <= 16, aligned): the sum ends in every lane
-template <int R>
-__device__ __forceinline__ float lanes_sum(float v) {
-  if (R >= 2) v = dpp_add_<0xB1>(v);    // quad_perm [1, 0, 3, 2]
-  if (R >= 4) v = dpp_add_<0x4E>(v);    // quad_perm [2, 3, 0, 1]
-  if (R >= 8) v = dpp_add_<0x141>(v);   // row_half_mirror
-  if (R >= 16) v = dpp_add_<0x140>(v);  // row_mirror
-  return v;
-}
-
 // ------------------------------------------------------------------------------------------------ selective scan
 // dt = softplus(dt_pre + bias);  S[c, n] <- exp(-dt_c e^{A_log[c, n]}) S[c, n] + dt_c x_c B_n;
 // y_c = sum_n S[c, n] C_n + D_c x_c;  out = scale * y * silu(z).
-// A lane owns NS states of CH channels; R = ceil(N / NS) lanes (a power of two <= 16) share those channels, a block of
-// 256 threads owns NC = 256 / R * CH channels of one sequence.  dt and dt x of the chunk go through LDS, a thread keeps
-// the x and z it fetched for the read-out of the same (token, channel) pairs.
-template <typename T, int NS, int R, int CH>
+// A lane owns NS states of CH = 2 channels; R >= N / NS lanes share those channels, a block of 256 threads owns
+// NC = 256 / R * CH channels of one sequence.  dt and dt x of the chunk go through LDS, a thread keeps the x and z it
+// fetched for the read-out of the same (token, channel) pairs.  Two tokens per turn: their four read-outs are summed over
+// the lanes together, and the next pair's inputs are read while the current pair is computed.
+constexpr int CH = 2;
+
+template <typename T, int NS, int R>
 __global__ __launch_bounds__(256) void k_selective_scan(const T* __restrict__ x, int ldx, const float* __restrict__ dtp,
                                                         const float* __restrict__ dtb, const T* __restrict__ bm, int ldb,
                                                         const T* __restrict__ cm, int ldc, const float* __restrict__ a_log,
@@ -74,40 +115,46 @@ __global__ __launch_bounds__(256) void k_selective_scan(const T* __restrict__ x,
                                                         int C, int N, SeqDesc d) {
   constexpr int NC = 256 / R * CH, PER = CT * NC / 256, NP = NS * R, PB = (CT * NP + 255) / 256;
   __shared__ __attribute__((aligned(16))) float sdt[CT * NC];
-  __shared__ __attribute__((aligned(16))) float sdx[CT * NC];     // dt x; the tokens' read-outs replace it
+  __shared__ __attribute__((aligned(16))) float sdx[CT * NC];     // dt x
+  __shared__ __attribute__((aligned(16))) float sy[CT * NC];      // the tokens' read-outs
   __shared__ __attribute__((aligned(16))) float sB[CT * NP];
   __shared__ __attribute__((aligned(16))) float sC[CT * NP];
   const int s = blockIdx.x, tid = threadIdx.x;
-  const int rg = tid % R, grp = tid / R, cb = blockIdx.y * NC, c0 = cb + grp * CH, n0 = rg * NS;
+  const int lane = tid & 63, grp = (tid >> 6) * (64 / R) + lane_group<R>(lane), row = lane >> 4;
+  const int cb = blockIdx.y * NC, c0 = cb + grp * CH, n0 = lane_part<R>(lane) * NS;
   if (d.live && !d.live[s]) return;
   const int t0 = d.seq_off[s], t1 = d.seq_off[s + 1], p0 = d.pos0[s], slot = d.slots[s];
   float Sr[CH][NS], A[CH][NS];
 #pragma unroll
   for (int h = 0; h < CH; ++h) {
     const bool ok = c0 + h < C;
-    const size_t row = ok ? c0 + h : 0;
-    load_state<NS>(a_log + row * N, n0, N, ok, A[h]);
-    load_state<NS>(S + ((size_t)slot * C + row) * N, n0, N, ok && p0 > 0, Sr[h]);
+    const size_t ch = ok ? c0 + h : 0;
+    load_state<NS>(a_log + ch * N, n0, N, ok, A[h]);
+    load_state<NS>(S + ((size_t)slot * C + ch) * N, n0, N, ok && p0 > 0, Sr[h]);
 #pragma unroll
     for (int i = 0; i < NS; ++i) A[h][i] = -expf(A[h][i]) * 1.4426950408889634f;    // decays as powers of two
   }
-  float fx[PER], fz[PER], fd[PER], gx[PER], gz[PER], fB[PB], fC[PB];
+  // A chunk's inputs are fetched without branches (addresses clamped to the step's last token and the last channel, values
+  // past them dropped when they are staged), so that all of a thread's loads are in flight together; a thread's channel
+  // is the same for all of its tokens.
+  static_assert(256 % NC == 0 && 256 % NP == 0, "a thread keeps its column");
+  const int fc = cb + tid % NC, ft = tid / NC, fcc = min(fc, C - 1), br = tid % NP, bt = tid / NP, brc = min(br, N - 1);
+  const float bias = dtb[fcc], skip = dskip[fcc];
+  T fx[PER], fz[PER], gx[PER], gz[PER], fB[PB], fC[PB];
+  float fd[PER];
   auto fetch = [&](int tb) {
-    const int n = min(CT, t1 - tb);
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
-      const int e = tid + 256 * i, tt = e / NC, c = cb + e % NC;
-      const bool ok = tt < n && c < C;
-      fx[i] = ok ? (float)x[(size_t)(tb + tt) * ldx + c] : 0.f;
-      fz[i] = ok ? (float)z[(size_t)(tb + tt) * ldz + c] : 0.f;
-      fd[i] = ok ? dtp[(size_t)(tb + tt) * C + c] + dtb[c] : 0.f;
+      const size_t t = min(tb + ft + 256 / NC * i, t1 - 1);
+      fx[i] = x[t * ldx + fcc];
+      fz[i] = z[t * ldz + fcc];
+      fd[i] = dtp[t * C + fcc];
     }
 #pragma unroll
     for (int i = 0; i < PB; ++i) {
-      const int e = tid + 256 * i, tt = e / NP, r = e % NP;
-      const bool ok = e < CT * NP && tt < n && r < N;
-      fB[i] = ok ? (float)bm[(size_t)(tb + tt) * ldb + r] : 0.f;
-      fC[i] = ok ? (float)cm[(size_t)(tb + tt) * ldc + r] : 0.f;
+      const size_t t = min(tb + bt + 256 / NP * i, t1 - 1);
+      fB[i] = bm[t * ldb + brc];
+      fC[i] = cm[t * ldc + brc];
     }
   };
   if (t0 < t1) fetch(t0);
@@ -116,55 +163,72 @@ __global__ __launch_bounds__(256) void k_selective_scan(const T* __restrict__ x,
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
-      const float dt = softplusf_(fd[i]);
+      const float dt = softplus_fast(fd[i] + bias);
       sdt[tid + 256 * i] = dt;
-      sdx[tid + 256 * i] = dt * fx[i];
+      sdx[tid + 256 * i] = dt * (float)fx[i];
       gx[i] = fx[i];
       gz[i] = fz[i];
     }
 #pragma unroll
     for (int i = 0; i < PB; ++i)
-      if (tid + 256 * i < CT * NP) {
-        sB[tid + 256 * i] = fB[i];
-        sC[tid + 256 * i] = fC[i];
+      if (CT * NP >= 256 || tid < CT * NP) {
+        sB[tid + 256 * i] = br < N ? (float)fB[i] : 0.f;          // a padded state never leaves zero
+        sC[tid + 256 * i] = br < N ? (float)fC[i] : 0.f;
       }
     __syncthreads();
     if (tb + CT < t1) fetch(tb + CT);
-    for (int tt = 0; tt < n; ++tt) {
-      float dt[CH], dx[CH], y[CH];
-#pragma unroll
-      for (int h = 0; h < CH; ++h) {
-        dt[h] = sdt[tt * NC + grp * CH + h];
-        dx[h] = sdx[tt * NC + grp * CH + h];
-        y[h] = 0.f;
-      }
+    struct In {
+      f32x4 B[NS / 4], C[NS / 4];
+      float dt[CH], dx[CH];
+    };
+    auto load = [&](int tt, In& in) {
 #pragma unroll
       for (int i4 = 0; i4 < NS / 4; ++i4) {
-        const f32x4 B = *reinterpret_cast<const f32x4*>(sB + tt * NP + n0 + 4 * i4);
-        const f32x4 Cv = *reinterpret_cast<const f32x4*>(sC + tt * NP + n0 + 4 * i4);
-#pragma unroll
-        for (int h = 0; h < CH; ++h)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const int i = 4 * i4 + j;
-            Sr[h][i] = __builtin_amdgcn_exp2f(dt[h] * A[h][i]) * Sr[h][i] + dx[h] * B[j];
-            y[h] += Sr[h][i] * Cv[j];
-          }
+        in.B[i4] = *reinterpret_cast<const f32x4*>(sB + tt * NP + n0 + 4 * i4);
+        in.C[i4] = *reinterpret_cast<const f32x4*>(sC + tt * NP + n0 + 4 * i4);
       }
 #pragma unroll
-      for (int h = 0; h < CH; ++h) y[h] = lanes_sum<R>(y[h]);
-      // (a channel's dt x is read only by the R lanes of its group, which run in lockstep: its place takes the read-out)
-      if (rg == 0)
+      for (int h = 0; h < CH; ++h) {
+        in.dt[h] = sdt[tt * NC + grp * CH + h];
+        in.dx[h] = sdx[tt * NC + grp * CH + h];
+      }
+    };
+    auto step = [&](const In& in, float (&y)[CH]) {
 #pragma unroll
-        for (int h = 0; h < CH; ++h) sdx[tt * NC + grp * CH + h] = y[h];
+      for (int h = 0; h < CH; ++h) {
+        float p[2] = {0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < NS; ++i) {
+          Sr[h][i] = __builtin_amdgcn_exp2f(in.dt[h] * A[h][i]) * Sr[h][i] + in.dx[h] * in.B[i >> 2][i & 3];
+          p[i & 1] += Sr[h][i] * in.C[i >> 2][i & 3];
+        }
+        y[h] = p[0] + p[1];
+      }
+    };
+    In a0, a1;
+    float ya[CH], yb[CH] = {0.f, 0.f};
+    load(0, a0);
+    int tt = 0;
+    for (; tt + 1 < n; tt += 2) {
+      load(tt + 1, a1);
+      step(a0, ya);
+      load(min(tt + 2, n - 1), a0);
+      step(a1, yb);
+      const float v = sum_four<R>(ya[0], ya[1], yb[0], yb[1]);     // row i of the wave: token tt + i / 2, channel i % 2
+      if (R == 4 || (lane & (R == 8 ? 1 : 3)) == 0) sy[(tt + (row >> 1)) * NC + grp * CH + (row & 1)] = v;
+    }
+    if (tt < n) {
+      step(a0, ya);
+      const float v = sum_four<R>(ya[0], ya[1], yb[0], yb[1]);
+      if ((R == 4 || (lane & (R == 8 ? 1 : 3)) == 0) && row < 2) sy[tt * NC + grp * CH + row] = v;
     }
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
-      const int e = tid + 256 * i, tt = e / NC, c = cb + e % NC;
-      if (tt < n && c < C) {
-        const float v = (sdx[e] + dskip[c] * gx[i]) * (gz[i] * sigmoidf_(gz[i])) * scale;
-        out[(size_t)(tb + tt) * ldo + c] = (T)v;
+      const int tt = ft + 256 / NC * i;
+      if (tt < n && fc < C) {
+        const float v = (sy[tid + 256 * i] + skip * (float)gx[i]) * silu_fast((float)gz[i]) * scale;
+        out[(size_t)(tb + tt) * ldo + fc] = (T)v;
       }
     }
   }
@@ -175,8 +239,9 @@ __global__ __launch_bounds__(256) void k_selective_scan(const T* __restrict__ x,
 
 // ------------------------------------------------------------------------------------------ gated linear attention
 // a = sigmoid(z + bias)^(1 / tau) per key channel;  S <- diag(a) S + k v^T;  o = S^T (qscale q).  S [slots, H, dv, dk].
-// A lane owns RR rows of CC = 4 columns; R lanes (a power of two <= 16) share those columns, a block of 256 threads owns
-// NC = 256 / R * 4 columns of one (sequence, head).  The decays are finished in float when a chunk is staged.
+// A lane owns RR rows of CC = 4 columns; R lanes share those columns, a block of 256 threads owns NC = 256 / R * 4 columns
+// of one (sequence, head).  The decays are finished in float when a chunk is staged; the next token's vectors are read
+// from LDS while the current token is computed.
 constexpr int CC = 4;
 
 template <typename T, int RR, int R>
@@ -189,31 +254,36 @@ __global__ __launch_bounds__(256) void k_gla_scan(const T* __restrict__ q, int l
   __shared__ __attribute__((aligned(16))) float sk[CT * DKP];
   __shared__ __attribute__((aligned(16))) float sq[CT * DKP];
   __shared__ __attribute__((aligned(16))) float sa[CT * DKP];
-  __shared__ __attribute__((aligned(16))) float sv[CT * NC];       // values; the tokens' read-outs replace them
+  __shared__ __attribute__((aligned(16))) float sv[CT * NC];
+  __shared__ __attribute__((aligned(16))) float so[CT * NC];       // the tokens' read-outs
   const int s = blockIdx.x / H, hd = blockIdx.x % H, cb = blockIdx.y * NC, tid = threadIdx.x;
   if (d.live && !d.live[s]) return;
-  const int rg = tid % R, grp = tid / R, c0 = cb + grp * CC, r0 = rg * RR;
+  const int lane = tid & 63, grp = (tid >> 6) * (64 / R) + lane_group<R>(lane), row = lane >> 4;
+  const int c0 = cb + grp * CC, r0 = lane_part<R>(lane) * RR;
   const int t0 = d.seq_off[s], t1 = d.seq_off[s + 1], p0 = d.pos0[s], slot = d.slots[s];
   float* Sh = S + ((size_t)slot * H + hd) * dv * dk;
   float Sr[CC][RR];
 #pragma unroll
   for (int c = 0; c < CC; ++c)
     load_state<RR>(Sh + (size_t)(c0 + c < dv ? c0 + c : 0) * dk, r0, dk, p0 > 0 && c0 + c < dv, Sr[c]);
-  float fk[PR], fq[PR], fz[PR], fv[PV];
-  auto fetch = [&](int tb) {
-    const int n = min(CT, t1 - tb);
+  static_assert(256 % NC == 0 && 256 % DKP == 0 && CT * DKP >= 256, "a thread keeps its row and its column");
+  const int fr = tid % DKP, frt = tid / DKP, frc = hd * dk + min(fr, dk - 1);
+  const int fc = cb + tid % NC, fct = tid / NC, fcc = hd * dv + min(fc, dv - 1);
+  const float bias = zb[frc];
+  T fk[PR], fq[PR], fv[PV];
+  float fz[PR];
+  auto fetch = [&](int tb) {                             // without branches, as in the selective scan
 #pragma unroll
     for (int i = 0; i < PR; ++i) {
-      const int e = tid + 256 * i, tt = e / DKP, r = e % DKP;
-      const bool ok = tt < n && r < dk;
-      fk[i] = ok ? (float)k[(size_t)(tb + tt) * ldk + hd * dk + r] : 0.f;
-      fq[i] = ok ? (float)q[(size_t)(tb + tt) * ldq + hd * dk + r] * qscale : 0.f;
-      fz[i] = ok ? z[(size_t)(tb + tt) * ((size_t)H * dk) + hd * dk + r] + zb[hd * dk + r] : 0.f;
+      const size_t t = min(tb + frt + 256 / DKP * i, t1 - 1);
+      fk[i] = k[t * ldk + frc];
+      fq[i] = q[t * ldq + frc];
+      fz[i] = z[t * ((size_t)H * dk) + frc];
     }
 #pragma unroll
     for (int i = 0; i < PV; ++i) {
-      const int e = tid + 256 * i, tt = e / NC, c = cb + e % NC;
-      fv[i] = tt < n && c < dv ? (float)v[(size_t)(tb + tt) * ldv + hd * dv + c] : 0.f;
+      const size_t t = min(tb + fct + 256 / NC * i, t1 - 1);
+      fv[i] = v[t * ldv + fcc];
     }
   };
   if (t0 < t1) fetch(t0);
@@ -221,43 +291,55 @@ __global__ __launch_bounds__(256) void k_gla_scan(const T* __restrict__ q, int l
     const int n = min(CT, t1 - tb);
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < PR; ++i)
-      if (tid + 256 * i < CT * DKP) {
-        sk[tid + 256 * i] = fk[i];
-        sq[tid + 256 * i] = fq[i];
-        sa[tid + 256 * i] = expf(logsigmoidf_(fz[i]) * inv_tau);
-      }
+    for (int i = 0; i < PR; ++i) {
+      sk[tid + 256 * i] = fr < dk ? (float)fk[i] : 0.f;       // a padded row never leaves zero
+      sq[tid + 256 * i] = fr < dk ? (float)fq[i] * qscale : 0.f;
+      const float zt = fz[i] + bias;                           // ln sigmoid(z) = min(z, 0) - ln(1 + e^-|z|)
+      sa[tid + 256 * i] = __builtin_amdgcn_exp2f((fminf(zt, 0.f) - log1p_exp_neg(fabsf(zt))) * (inv_tau * 1.4426950408889634f));
+    }
 #pragma unroll
-    for (int i = 0; i < PV; ++i) sv[tid + 256 * i] = fv[i];
+    for (int i = 0; i < PV; ++i) sv[tid + 256 * i] = (float)fv[i];
     __syncthreads();
     if (tb + CT < t1) fetch(tb + CT);
-    for (int tt = 0; tt < n; ++tt) {
-      const f32x4 vv = *reinterpret_cast<const f32x4*>(sv + tt * NC + grp * CC);
-      float o[CC] = {0.f, 0.f, 0.f, 0.f};
+    struct In {
+      f32x4 k[RR / 4], a[RR / 4], q[RR / 4], v;
+    };
+    auto load = [&](int tt, In& in) {
 #pragma unroll
       for (int i4 = 0; i4 < RR / 4; ++i4) {
-        const f32x4 kk = *reinterpret_cast<const f32x4*>(sk + tt * DKP + r0 + 4 * i4);
-        const f32x4 aa = *reinterpret_cast<const f32x4*>(sa + tt * DKP + r0 + 4 * i4);
-        const f32x4 qq = *reinterpret_cast<const f32x4*>(sq + tt * DKP + r0 + 4 * i4);
-#pragma unroll
-        for (int c = 0; c < CC; ++c)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const int i = 4 * i4 + j;
-            Sr[c][i] = aa[j] * Sr[c][i] + kk[j] * vv[c];
-            o[c] += Sr[c][i] * qq[j];
-          }
+        in.k[i4] = *reinterpret_cast<const f32x4*>(sk + tt * DKP + r0 + 4 * i4);
+        in.a[i4] = *reinterpret_cast<const f32x4*>(sa + tt * DKP + r0 + 4 * i4);
+        in.q[i4] = *reinterpret_cast<const f32x4*>(sq + tt * DKP + r0 + 4 * i4);
       }
+      in.v = *reinterpret_cast<const f32x4*>(sv + tt * NC + grp * CC);
+    };
+    auto step = [&](int tt, const In& in) {
+      float o[CC] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int c = 0; c < CC; ++c) o[c] = lanes_sum<R>(o[c]);
-      // (the four values are read only by this group of lanes, which run in lockstep: their place takes the read-out)
-      if (rg == 0) *reinterpret_cast<f32x4*>(sv + tt * NC + grp * CC) = f32x4{o[0], o[1], o[2], o[3]};
+      for (int i = 0; i < RR; ++i)
+#pragma unroll
+        for (int c = 0; c < CC; ++c) {
+          Sr[c][i] = in.a[i >> 2][i & 3] * Sr[c][i] + in.k[i >> 2][i & 3] * in.v[c];
+          o[c] += Sr[c][i] * in.q[i >> 2][i & 3];
+        }
+      const float v = sum_four<R>(o[0], o[1], o[2], o[3]);          // row c of the wave: column c
+      if (R == 4 || (lane & (R == 8 ? 1 : 3)) == 0) so[tt * NC + grp * CC + row] = v;
+    };
+    In a0, a1;
+    load(0, a0);
+    int tt = 0;
+    for (; tt + 1 < n; tt += 2) {
+      load(tt + 1, a1);
+      step(tt, a0);
+      load(min(tt + 2, n - 1), a0);
+      step(tt + 1, a1);
     }
+    if (tt < n) step(tt, a0);
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < PV; ++i) {
-      const int e = tid + 256 * i, tt = e / NC, c = cb + e % NC;
-      if (tt < n && c < dv) out[((size_t)(tb + tt) * H + hd) * dv + c] = sv[e];
+      const int tt = fct + 256 / NC * i;
+      if (tt < n && fc < dv) out[((size_t)(tb + tt) * H + hd) * dv + fc] = so[tid + 256 * i];
     }
   }
 #pragma unroll
@@ -274,25 +356,21 @@ void seq_selective_scan(int code, const void* x, int ldx, const float* dtp, cons
                         const void* c, int ldc, const float* a_log, const float* dskip, const void* z, int ldz, float* S,
                         void* out, int ldo, float scale, int C, int N, SeqDesc d, hipStream_t st) {
   if (d.B == 0) return;
-#define SEL_LAUNCH(NS_, R_, CH_)                                                                                           \
-  hipLaunchKernelGGL((k_selective_scan<T, NS_, R_, CH_>), dim3(d.B, (C + 256 / R_ * CH_ - 1) / (256 / R_ * CH_)), dim3(256), \
+#define SEL_LAUNCH(NS_, R_)                                                                                           \
+  hipLaunchKernelGGL((k_selective_scan<T, NS_, R_>), dim3(d.B, (C + 256 / R_ * CH - 1) / (256 / R_ * CH)), dim3(256), \
                      0, st, (const T*)x, ldx, dtp, dtb, (const T*)b, ldb, (const T*)c, ldc, a_log, dskip, (const T*)z, ldz, \
                      S, (T*)out, ldo, scale, C, N, d)
   SEQ_DISPATCH_T(code, {
-    if (N <= 4)
-      SEL_LAUNCH(4, 1, 1);
-    else if (N <= 8)
-      SEL_LAUNCH(4, 2, 1);
-    else if (N <= 16)
-      SEL_LAUNCH(4, 4, 2);
+    if (N <= 16)
+      SEL_LAUNCH(4, 4);
     else if (N <= 32)
-      SEL_LAUNCH(4, 8, 2);
+      SEL_LAUNCH(4, 8);
     else if (N <= 64)
-      SEL_LAUNCH(4, 16, 2);
+      SEL_LAUNCH(4, 16);
     else if (N <= 128)
-      SEL_LAUNCH(8, 16, 1);
+      SEL_LAUNCH(8, 16);
     else
-      SEL_LAUNCH(16, 16, 1);
+      SEL_LAUNCH(16, 16);
   });
 #undef SEL_LAUNCH
   LIPA_CHECK_LAUNCH();
