@@ -125,14 +125,20 @@ __device__ __forceinline__ bf16x4 tr_read(const bf16* p) {
 
 // NW = 4 puts four query heads of one kv head (and one value head c) into a block: the key and value tiles are loaded
 // once into LDS for the four waves instead of once per head.
-template <int NDS, int NDT, bool HEADS, int NW, bool GQA>
-__global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ kc,
+//
+// EXACT: dk = 16 NDS and dv = 32 NDT, and no distance bias; every loop has constant bounds and no score meets a branch:
+// tiles that every query sees whole skip the masks, the output is rescaled only when a maximum has moved, and the next
+// tile's keys and values (one wave: all of them in registers) are fetched while the current tile is computed.  CAP
+// (EXACT only): scores are bounded.
+template <int NDS, int NDT, bool HEADS, int NW, bool GQA, bool EXACT, bool CAP>
+__global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ kc,
                                                        const bf16* __restrict__ vc, float* __restrict__ pm,
                                                        float* __restrict__ pl, float* __restrict__ pu,
                                                        const int* __restrict__ tile_seq, const int* __restrict__ tile_t0,
-                                                       int H, int G, int dk, int dv, int ldk, int ldv, int max_len,
+                                                       int H, int G, int dk_, int dv_, int ldk, int ldv, int max_len,
                                                        int nsplit, float scale, SeqDesc d, GqaExtra x) {
   constexpr int LDMAX = NDT * 32 + 8, LDKMAX = NDS * 16 + 8;
+  const int dk = EXACT ? NDS * 16 : dk_, dv = EXACT ? NDT * 32 : dv_;
   __shared__ __attribute__((aligned(16))) bf16 sV[32 * LDMAX];
   __shared__ __attribute__((aligned(16))) bf16 sK[NW > 1 ? 32 * LDKMAX : 8];
   const int tile = blockIdx.x, z = GQA ? blockIdx.z : blockIdx.z / G;
@@ -151,13 +157,16 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
     lo_t = max(lo_t, (HEADS ? pos_q : d.tok_pos[t0]) - win + 1);
     lo_q = max(lo_q, pos_q - win + 1);
   }
-  const float* brow = (GQA && x.bias != nullptr) ? x.bias + (size_t)g * x.nd : nullptr;
+  const float* brow = (!EXACT && GQA && x.bias != nullptr) ? x.bias + (size_t)g * x.nd : nullptr;
   // a tile's queries sit at consecutive positions p0 + ql, so a 32-key tile meets only the 63 distances
   // p0 - jb - 31 + i: lane i fetches that one bias and the 16 a lane needs come from its neighbours' registers
   const int p0 = HEADS ? pos_q : d.tok_pos[t0];
   const float sl2 = scale * 1.4426950408889634f;   // scores in units of log2: v_exp_f32 is 2^x
   // bounded scores: cap tanh(u) = cap - 2 cap / (e^2u + 1), with e^2u as a power of two
-  const float cap = GQA ? x.softcap : 0.f, cl2 = cap * 1.4426950408889634f, ce = cap > 0.f ? 2.f * sl2 / cap : 0.f;
+  const bool capped = EXACT ? CAP : GQA && x.softcap > 0.f;
+  const float cl2 = x.softcap * 1.4426950408889634f, ce = capped ? 2.f * sl2 / x.softcap : 0.f;
+  // from this key on every query of the tile sees a key that is not in its future
+  const int lo_all = EXACT ? (blk > 0 ? (pmax / blk) * blk : win > 0 ? pmax - win + 1 : 0) : 0;
   const int trow = 4 * (lane >> 5) + ((lane & 15) >> 2), tcol = 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
   const int per = (pmax - lo_t + nsplit) / nsplit, j0 = lo_t + z * per, j1 = min(pmax + 1, j0 + per);
   const bf16* kbase = kc + ((size_t)slot * max_len) * ldk + kh * dk + 8 * hi;
@@ -165,7 +174,7 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
   bf16x8 qf[NDS];
 #pragma unroll
   for (int ds = 0; ds < NDS; ++ds)
-    if (ds < nds) qf[ds] = *reinterpret_cast<const bf16x8*>(q + (size_t)tq * ldq + g * dk + 16 * ds + 8 * hi);
+    if (EXACT || ds < nds) qf[ds] = *reinterpret_cast<const bf16x8*>(q + (size_t)tq * ldq + g * dk + 16 * ds + 8 * hi);
   f32x16 acc[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
@@ -173,39 +182,41 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
     for (int r = 0; r < 16; ++r) acc[dt][r] = 0.f;
   float m = -INFINITY, l = 0.f;
   const int vpr = dv >> 3, kpr = dk >> 3;        // 16 B vectors per value / key row
-  // four waves: the next key / value tile is fetched into registers while the current one is computed on
-  constexpr int VPT = NW > 1 ? (2 * NDT) / NW : 1, KPT = NW > 1 ? (2 * NDS) / NW : 1;
+  // the next key / value tile is fetched into registers while the current one is computed on (one wave: EXACT only, and
+  // the keys come straight in the operand layout)
+  constexpr bool AHEAD = NW > 1 || EXACT;
+  constexpr int VPT = AHEAD ? (2 * NDT + NW - 1) / NW : 1, KPT = NW > 1 ? (NDS + NW - 1) / NW : EXACT ? NDS : 1;
   bf16x8 pv[VPT], pk[KPT];
   auto fetch = [&](int jb) {
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
       const int e = threadIdx.x + 64 * NW * i, row = e / vpr, cv = e % vpr;
-      if (e < 32 * vpr)
+      if ((EXACT && (2 * NDT) % NW == 0) || e < 32 * vpr)
         pv[i] = *reinterpret_cast<const bf16x8*>(vbase + (size_t)min(jb + row, max_len - 1) * ldv + cv * 8);
+    }
+    if (NW == 1) {
+#pragma unroll
+      for (int i = 0; i < KPT; ++i)
+        pk[i] = *reinterpret_cast<const bf16x8*>(kbase + (size_t)min(jb + ql, max_len - 1) * ldk + 16 * i);
+      return;
     }
 #pragma unroll
     for (int i = 0; i < KPT; ++i) {
       const int e = threadIdx.x + 64 * NW * i, row = e / kpr, cv = e % kpr;
-      if (e < 32 * kpr)
+      if ((EXACT && NDS % NW == 0) || e < 32 * kpr)
         pk[i] = *reinterpret_cast<const bf16x8*>(kbase - 8 * hi + (size_t)min(jb + row, max_len - 1) * ldk + cv * 8);
     }
   };
-  if (NW > 1 && j0 < j1) fetch(j0);
+  if (AHEAD && j0 < j1) fetch(j0);
   for (int jb = j0; jb < j1; jb += 32) {
     __syncthreads();
-    if (NW > 1) {
+    if (AHEAD) {
 #pragma unroll
       for (int i = 0; i < VPT; ++i) {
         const int e = threadIdx.x + 64 * NW * i;
-        if (e < 32 * vpr) *reinterpret_cast<bf16x8*>(sV + (e / vpr) * LD + (e % vpr) * 8) = pv[i];
+        if ((EXACT && (2 * NDT) % NW == 0) || e < 32 * vpr)
+          *reinterpret_cast<bf16x8*>(sV + (e / vpr) * LD + (e % vpr) * 8) = pv[i];
       }
-#pragma unroll
-      for (int i = 0; i < KPT; ++i) {
-        const int e = threadIdx.x + 64 * NW * i;
-        if (e < 32 * kpr) *reinterpret_cast<bf16x8*>(sK + (e / kpr) * LDK + (e % kpr) * 8) = pk[i];
-      }
-      __syncthreads();
-      if (jb + 32 < j1) fetch(jb + 32);
     } else {
       for (int e = threadIdx.x; e < 32 * vpr; e += 64) {
         const int row = e / vpr, cv = e % vpr;
@@ -213,27 +224,53 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
             *reinterpret_cast<const bf16x8*>(vbase + (size_t)min(jb + row, max_len - 1) * ldv + cv * 8);
       }
     }
+    if (NW > 1) {
+#pragma unroll
+      for (int i = 0; i < KPT; ++i) {
+        const int e = threadIdx.x + 64 * NW * i;
+        if ((EXACT && NDS % NW == 0) || e < 32 * kpr)
+          *reinterpret_cast<bf16x8*>(sK + (e / kpr) * LDK + (e % kpr) * 8) = pk[i];
+      }
+      __syncthreads();
+      if (jb + 32 < j1) fetch(jb + 32);
+    }
     f32x16 sc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) sc[r] = 0.f;
-    const bf16* kr = NW > 1 ? sK + ql * LDK + 8 * hi : kbase + (size_t)min(jb + ql, max_len - 1) * ldk;
+    if (EXACT && NW == 1) {
 #pragma unroll
-    for (int ds = 0; ds < NDS; ++ds)
-      if (ds < nds)
-        sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(kr + 16 * ds), qf[ds], sc, 0, 0, 0);
+      for (int ds = 0; ds < NDS; ++ds) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pk[ds < KPT ? ds : 0], qf[ds], sc, 0, 0, 0);
+      if (jb + 32 < j1) fetch(jb + 32);
+    } else {
+      const bf16* kr = NW > 1 ? sK + ql * LDK + 8 * hi : kbase + (size_t)min(jb + ql, max_len - 1) * ldk;
+#pragma unroll
+      for (int ds = 0; ds < NDS; ++ds)
+        if (EXACT || ds < nds)
+          sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(kr + 16 * ds), qf[ds], sc, 0, 0, 0);
+    }
     float mt = -INFINITY, bw = 0.f;
-    if (GQA && !HEADS && brow != nullptr)
+    if (!EXACT && GQA && !HEADS && brow != nullptr)
       bw = brow[min(max(p0 - jb - 31 + lane, 0), x.nd - 1)] * 1.4426950408889634f;
+    auto score = [&](float a) {
+      return capped ? cl2 - 2.f * cl2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(a * ce) + 1.f) : a * sl2;
+    };
+    if (EXACT && jb + 31 <= p0 && jb + 32 <= j1 && jb >= lo_all) {      // every query sees the whole tile
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const int kk = (r & 3) + 8 * (r >> 2) + 4 * hi, key = jb + kk;
-      const bool seen = key <= pos_q && key < j1 && (!GQA || key >= lo_q);
-      float v = sc[r] * sl2;
-      if (GQA && cap > 0.f) v = cl2 - 2.f * cl2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[r] * ce) + 1.f);
-      if (GQA && !HEADS && brow != nullptr) v += __shfl(bw, ql - kk + 31, 64);
-      if (GQA && HEADS && brow != nullptr && seen) v += brow[min(pos_q - key, x.nd - 1)] * 1.4426950408889634f;
-      sc[r] = seen ? v : -INFINITY;
-      mt = fmaxf(mt, sc[r]);
+      for (int r = 0; r < 16; ++r) {
+        sc[r] = score(sc[r]);
+        mt = fmaxf(mt, sc[r]);
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int kk = (r & 3) + 8 * (r >> 2) + 4 * hi, key = jb + kk;
+        const bool seen = key <= pos_q && key < j1 && (!GQA || key >= lo_q);
+        float v = score(sc[r]);
+        if (!EXACT && GQA && !HEADS && brow != nullptr) v += __shfl(bw, ql - kk + 31, 64);
+        if (!EXACT && GQA && HEADS && brow != nullptr && seen) v += brow[min(pos_q - key, x.nd - 1)] * 1.4426950408889634f;
+        sc[r] = seen ? v : -INFINITY;
+        mt = fmaxf(mt, sc[r]);
+      }
     }
     mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
     const float mn = fmaxf(m, mt), ms = mn == -INFINITY ? 0.f : mn;
@@ -246,11 +283,13 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
     }
     rs += __shfl_xor(rs, 32, 64);
     l = l * corr + rs;
+    if (!EXACT || __any(mn > m)) {                 // (a maximum that has not moved leaves the output as it is)
+#pragma unroll
+      for (int dt = 0; dt < NDT; ++dt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) acc[dt][r] *= corr;
+    }
     m = mn;
-#pragma unroll
-    for (int dt = 0; dt < NDT; ++dt)
-#pragma unroll
-      for (int r = 0; r < 16; ++r) acc[dt][r] *= corr;
     if (NW == 1) __syncthreads();                  // (four waves: the barrier after the tile copies covers V too)
 #pragma unroll
     for (int u2 = 0; u2 < 2; ++u2) {
@@ -259,7 +298,7 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
       for (int j = 0; j < 8; ++j) pb[j] = (bf16)sc[8 * u2 + j];
 #pragma unroll
       for (int dt = 0; dt < NDT; ++dt)
-        if (dt < ndt) {
+        if (EXACT || dt < ndt) {
           // transposing LDS reads: the 16 lanes of a group address a 4-key x 16-column block (lane 4q'+p': key q',
           // columns 4p'..4p'+3) and lane i receives column i's four keys; keys 16u2 + 4hi + 0..3, then the same + 8
           const bf16* vp = sV + (16 * u2 + trow) * LD + dt * 32 + tcol;
@@ -280,17 +319,17 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
       const bf16* grow = (const bf16*)x.gate + (size_t)tq * x.ldg + g * dv;
 #pragma unroll
       for (int dt = 0; dt < NDT; ++dt)
-        if (dt < ndt)
+        if (EXACT || dt < ndt)
 #pragma unroll
           for (int r4 = 0; r4 < 4; ++r4) {
             const bf16x4 gv = *reinterpret_cast<const bf16x4*>(grow + dt * 32 + 8 * r4 + 4 * hi);
 #pragma unroll
-            for (int j = 0; j < 4; ++j) acc[dt][4 * r4 + j] *= sigmoidf_((float)gv[j]);
+            for (int j = 0; j < 4; ++j) acc[dt][4 * r4 + j] *= __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f((float)gv[j] * -1.4426950408889634f));
           }
     }
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt)
-      if (dt < ndt)
+      if (EXACT || dt < ndt)
 #pragma unroll
         for (int r4 = 0; r4 < 4; ++r4)
           *reinterpret_cast<bf16x4*>(orow + dt * 32 + 8 * r4 + 4 * hi) =
@@ -305,7 +344,7 @@ __global__ __launch_bounds__(64 * NW) void k_talk_attn_mfma(const bf16* __restri
   }
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
-    if (dt < ndt)
+    if (EXACT || dt < ndt)
 #pragma unroll
       for (int r4 = 0; r4 < 4; ++r4)
         *reinterpret_cast<f32x4*>(pu + o * GV + (GQA ? 0 : c * dv) + dt * 32 + 8 * r4 + 4 * hi) =
@@ -371,23 +410,39 @@ static bool sweep(int code, const void* q, int ldq, const void* kc, int ldk, con
     const bool heads = ntiles == d.Ttot && H / G <= 32 && H / G > 1;    // one token per tile: group the heads instead
     const int nw = (!heads && (H / G) % 4 == 0) ? 4 : 1;                 // four heads of a kv head share its tiles
     const dim3 grid(ntiles, heads ? G : H / nw, GQA ? nsplit : G * nsplit);
-#define SEQ_ATTN_LAUNCH(NDS, NDT, HEADS, NW)                                                                        \
-  hipLaunchKernelGGL((k_talk_attn_mfma<NDS, NDT, HEADS, NW, GQA>), grid, dim3(64 * NW), 0, st, (const bf16*)q, ldq,  \
-                     (const bf16*)kc, (const bf16*)vc, pm, pl, pu, tile_seq, tile_t0, H, G, dk, dv, ldk, ldv, max_len, \
+#define SEQ_ATTN_LAUNCH(NDS, NDT, HEADS, NW, EXACT, CAP)                                                              \
+  hipLaunchKernelGGL((k_talk_attn_mfma<NDS, NDT, HEADS, NW, GQA, EXACT, CAP>), grid, dim3(64 * NW), 0, st, (const bf16*)q, \
+                     ldq, (const bf16*)kc, (const bf16*)vc, pm, pl, pu, tile_seq, tile_t0, H, G, dk, dv, ldk, ldv, max_len, \
                      nsplit, scale, d, x)
-    bool small = false;                            // small heads: half the accumulators, more waves per SIMD
+#define SEQ_ATTN_FORMS(NDS, NDT, EXACT, CAP)                                                   \
+  do {                                                                                        \
+    if (heads) SEQ_ATTN_LAUNCH(NDS, NDT, true, 1, EXACT, CAP);                                \
+    else if (nw == 4) SEQ_ATTN_LAUNCH(NDS, NDT, false, 4, EXACT, CAP);                        \
+    else SEQ_ATTN_LAUNCH(NDS, NDT, false, 1, EXACT, CAP);                                     \
+  } while (0)
+#define SEQ_ATTN_EXACT(NDS, NDT)                                                              \
+  do {                                                                                        \
+    if (x.softcap > 0.f) SEQ_ATTN_FORMS(NDS, NDT, true, true);                                \
+    else SEQ_ATTN_FORMS(NDS, NDT, true, false);                                               \
+  } while (0)
+    bool done = false;
     if constexpr (GQA) {
-      small = dk <= 64 && dv <= 64;
-      if (small) {
-        if (heads) SEQ_ATTN_LAUNCH(4, 2, true, 1); else if (nw == 4) SEQ_ATTN_LAUNCH(4, 2, false, 4); else SEQ_ATTN_LAUNCH(4, 2, false, 1);
+      if (x.bias == nullptr && dk == dv && (dk == 64 || dk == 96 || dk == 128)) {
+        if (dk == 64) SEQ_ATTN_EXACT(4, 2); else if (dk == 96) SEQ_ATTN_EXACT(6, 3); else SEQ_ATTN_EXACT(8, 4);
+        done = true;
+      } else if (dk <= 64 && dv <= 64) {           // small heads: half the accumulators, more waves per SIMD
+        SEQ_ATTN_FORMS(4, 2, false, false);
+        done = true;
       }
     }
-    if (small) {
+    if (done) {
     } else if (dk <= 128 && dv <= 128) {
-      if (heads) SEQ_ATTN_LAUNCH(8, 4, true, 1); else if (nw == 4) SEQ_ATTN_LAUNCH(8, 4, false, 4); else SEQ_ATTN_LAUNCH(8, 4, false, 1);
+      SEQ_ATTN_FORMS(8, 4, false, false);
     } else {
-      if (heads) SEQ_ATTN_LAUNCH(16, 8, true, 1); else if (nw == 4) SEQ_ATTN_LAUNCH(16, 8, false, 4); else SEQ_ATTN_LAUNCH(16, 8, false, 1);
+      SEQ_ATTN_FORMS(16, 8, false, false);
     }
+#undef SEQ_ATTN_EXACT
+#undef SEQ_ATTN_FORMS
 #undef SEQ_ATTN_LAUNCH
     LIPA_CHECK_LAUNCH();
     return GQA && nsplit == 1;
@@ -411,40 +466,47 @@ void seq_attn_sweep(int code, const void* q, int ldq, const void* kc, int ldk, c
                ntiles, d, GqaExtra{nullptr, 0, 0, 0, 0.f, nullptr, 0, nullptr, 0, 1.f, 0.f, nullptr, 0}, st);
 }
 
-// Merge of a GQA sweep's key splits: one wave per (token, head); the sink joins the denominator here.
+// Merge of a GQA sweep's key splits: one block of four waves per (token, head), a wave takes every fourth split, so the
+// loads of a few dozen splits are in flight together; the sink joins the denominator here.
 template <typename T>
-__global__ __launch_bounds__(64) void k_gqa_merge(const float* __restrict__ pm, const float* __restrict__ pl,
-                                                  const float* __restrict__ pu, T* __restrict__ out, int H, int dv,
-                                                  int nsplit, int sink, float sink_logit,
-                                                  const float* __restrict__ sinks, int ldo, float out_scale,
-                                                  const T* __restrict__ gate, int ldg) {
-  const int t = blockIdx.x, g = blockIdx.y, lane = threadIdx.x;
+__global__ __launch_bounds__(256) void k_gqa_merge(const float* __restrict__ pm, const float* __restrict__ pl,
+                                                   const float* __restrict__ pu, T* __restrict__ out, int H, int dv,
+                                                   int nsplit, int sink, float sink_logit,
+                                                   const float* __restrict__ sinks, int ldo, float out_scale,
+                                                   const T* __restrict__ gate, int ldg) {
+  __shared__ float part[4 * 64];
+  __shared__ float sw[1024];                         // a split's weight (nsplit <= 1024)
+  const int t = blockIdx.x, g = blockIdx.y, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const size_t b = ((size_t)t * H + g) * nsplit;
   if (sinks != nullptr) sink_logit = sinks[g];
-  // a lane takes split z = lane (+ 64 ...): maximum and denominator are wave reductions, a split's weight is handed round
+  // every wave finds the maximum and the denominator by itself
   float mx = sink ? sink_logit : -INFINITY;
   for (int z = lane; z < nsplit; z += 64) mx = fmaxf(mx, pm[b + z]);
   mx = wave_max(mx);
   float l = 0.f;
-  for (int z = lane; z < nsplit; z += 64) l += pm[b + z] == -INFINITY ? 0.f : expf(pm[b + z] - mx) * pl[b + z];
+  for (int z = lane; z < nsplit; z += 64) {
+    const float mz = pm[b + z], w = mz == -INFINITY ? 0.f : expf(mz - mx);
+    l += w * pl[b + z];
+    if (wv == 0) sw[z] = w;
+  }
   l = wave_sum(l) + (sink ? expf(sink_logit - mx) : 0.f);
   const float inv = l > 0.f ? out_scale / l : 0.f;
+  __syncthreads();
   for (int c0 = 0; c0 < dv; c0 += 64) {
     const int col = c0 + lane;
     float u = 0.f;
-    for (int z0 = 0; z0 < nsplit; z0 += 64) {
-      const int nz = min(64, nsplit - z0);
-      const float mz = lane < nz ? pm[b + z0 + lane] : -INFINITY;
-      const float wz = mz == -INFINITY ? 0.f : expf(mz - mx);
+    if (col < dv) {
 #pragma unroll 8
-      for (int z = 0; z < nz; ++z) {
-        const float w = __shfl(wz, z, 64);            // (an empty split has weight 0; its sums were written as 0)
-        if (col < dv) u += w * pu[(b + z0 + z) * dv + col];
-      }
+      for (int z = wv; z < nsplit; z += 4) u += sw[z] * pu[(b + z) * dv + col];
     }
-    if (col >= dv) continue;
-    if (gate != nullptr) u *= sigmoidf_((float)gate[(size_t)t * ldg + g * dv + col]);
-    out[(size_t)t * ldo + g * dv + col] = (T)(u * inv);
+    part[wv * 64 + lane] = u;
+    __syncthreads();
+    if (wv == 0 && col < dv) {
+      u = (part[lane] + part[64 + lane]) + (part[128 + lane] + part[192 + lane]);
+      if (gate != nullptr) u *= sigmoidf_((float)gate[(size_t)t * ldg + g * dv + col]);
+      out[(size_t)t * ldo + g * dv + col] = (T)(u * inv);
+    }
+    __syncthreads();
   }
 }
 
@@ -462,7 +524,7 @@ void seq_gqa_attention(int code, const void* q, int ldq, const void* kc, int ldk
                                   GqaExtra{bias, nd, block, sink, sink_logit, out, window, sinks, ldo, out_scale, softcap,
                                            gate, ldg}, st);
   if (direct) return;
-  SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_gqa_merge<T>, dim3(d.Ttot, H), dim3(64), 0, st, pm, pl, pu, (T*)out, H, dv,
+  SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_gqa_merge<T>, dim3(d.Ttot, H), dim3(256), 0, st, pm, pl, pu, (T*)out, H, dv,
                                           nsplit, sink, sink_logit, sinks, ldo, out_scale, (const T*)gate, ldg));
   LIPA_CHECK_LAUNCH();
 }
