@@ -511,6 +511,71 @@ __global__ __launch_bounds__(256) void k_rope_kv_store(const T* __restrict__ u, 
     for (int c = threadIdx.x; c < nv; c += 256) vc[row * nv + c] = r[nq + nk + c];
 }
 
+// The same, four entries per thread (16-byte or 8-byte accesses; dk and dv multiples of 4, dims of 8 when `half`).
+template <typename T>
+__global__ __launch_bounds__(256) void k_rope_kv_store4(const T* __restrict__ u, int ldu, const float* __restrict__ inv_freq,
+                                                        T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
+                                                        int nq, int nk, int nv, int dk, int dims, int half, float mag,
+                                                        int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
+                                                        SeqDesc d) {
+  const size_t t = blockIdx.x;
+  const T* r = u + t * ldu;
+  const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]], hd = dims >> 1;
+  const float p = (float)pos;
+  const float temp = tevery > 0 && pos >= 0 ? 1.f + tcoef * logf((float)((pos + 1) / tevery + 1)) : 1.f;
+  const bool keep = pos >= 0 && pos < max_len;       // a row nobody reads may carry any position
+  const size_t row = (size_t)slot * max_len + (keep ? pos : 0);
+  for (int c = 4 * threadIdx.x; c < nq + nk; c += 1024) {
+    const bool isq = c < nq;
+    if (!isq && !keep) break;
+    const int cl = c % dk;
+    const f32x4 a = load4_act<T>(r + c);
+    f32x4 o = a;
+    if (cl < dims) {
+      if (half) {
+        const bool second = cl >= hd;
+        const f32x4 b = load4_act<T>(r + (second ? c - hd : c + hd));
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          float sn, cs;
+          sincosf(p * inv_freq[(second ? cl - hd : cl) + j], &sn, &cs);
+          o[j] = (second ? a[j] * cs + b[j] * sn : a[j] * cs - b[j] * sn) * mag;
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; j += 2)
+          if (cl + j < dims) {
+            float sn, cs;
+            sincosf(p * inv_freq[(cl + j) >> 1], &sn, &cs);
+            o[j] = (a[j] * cs - a[j + 1] * sn) * mag;
+            o[j + 1] = (a[j + 1] * cs + a[j] * sn) * mag;
+          }
+      }
+    }
+    if (isq)
+      store4_act(qout + t * nq + c, o * temp);
+    else {
+      store4_act(kc + row * nk + c - nq, o);
+      if (vkeys && veps < 0.f) store4_act(vc + row * nk + c - nq, a);
+    }
+  }
+  if (!keep) return;
+  const T* vr = r + (vkeys ? nq : nq + nk);
+  if (veps >= 0.f) {                                 // one wave per head: the value over its root mean square
+    const int lane = threadIdx.x & 63;
+    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
+      float ss = 0.f;
+      for (int c = 4 * lane; c < dv; c += 256) {
+        const f32x4 v = load4_act<T>(vr + h0 + c);
+        ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+      }
+      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
+      for (int c = 4 * lane; c < dv; c += 256) store4_act(vc + row * nv + h0 + c, load4_act<T>(vr + h0 + c) * rs);
+    }
+  } else if (!vkeys)
+    for (int c = 4 * threadIdx.x; c < nv; c += 1024) store4_act(vc + row * nv + c, load4_act<T>(vr + c));
+}
+
 // out = y * sigmoid(gate), element by element; gate rows are ldg apart
 template <typename T>
 __global__ __launch_bounds__(256) void k_sigmoid_gate(const T* __restrict__ y, const T* __restrict__ gate, int ldg,
@@ -598,6 +663,14 @@ void seq_rope_kv_store(int code, const void* u, int ldu, const float* inv_freq, 
                        int nk, int nv, int dk, int dims, int half, float mag, int vkeys, int max_len, float tcoef,
                        int tevery, float veps, int dv, SeqDesc d, hipStream_t st) {
   if (d.Ttot == 0) return;
+  const bool vec = ldu % 4 == 0 && dk % 4 == 0 && dv % 4 == 0 && (!half || dims % 8 == 0) && ((uintptr_t)u & 15) == 0;
+  if (vec) {
+    SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_rope_kv_store4<T>, dim3(d.Ttot), dim3(256), 0, st, (const T*)u, ldu, inv_freq,
+                                            (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef,
+                                            tevery, veps, dv, d));
+    LIPA_CHECK_LAUNCH();
+    return;
+  }
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_rope_kv_store<T>, dim3(d.Ttot), dim3(256), 0, st, (const T*)u, ldu, inv_freq,
                                           (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef,
                                           tevery, veps, dv, d));

@@ -117,7 +117,9 @@ __global__ __launch_bounds__(64) void k_conv_run(const T* __restrict__ u, int ld
     for (int i = 0; i < 4; ++i) cw[j][i] = j >= TP - taps ? w[(size_t)(c + i) * taps + j - (TP - taps)] : 0.f;
   if (bias != nullptr) b = conv_ld4(bias + c);
   int cur = -1, slot = 0;
+  f32x4 x = conv_ld4(u + (size_t)t0 * ldu + c);
   for (int t = t0; t < t1; ++t) {
+    const f32x4 xn = conv_ld4(u + (size_t)min(t + 1, t1 - 1) * ldu + c);       // in flight while this token is computed
     const int s = d.tok_seq[t];
     if (s != cur) {
       cur = s;
@@ -135,7 +137,6 @@ __global__ __launch_bounds__(64) void k_conv_run(const T* __restrict__ u, int ld
         }
       }
     }
-    const f32x4 x = conv_ld4(u + (size_t)t * ldu + c);
     f32x4 y = b + cw[TP - 1] * x;
 #pragma unroll
     for (int j = 0; j < TP - 1; ++j) y += cw[j] * win[j];
@@ -146,6 +147,7 @@ __global__ __launch_bounds__(64) void k_conv_run(const T* __restrict__ u, int ld
 #pragma unroll
     for (int j = 0; j < TP - 2; ++j) win[j] = win[j + 1];
     win[TP - 2] = x;
+    x = xn;
     if (roll && !(d.live && !d.live[s]))
 #pragma unroll
       for (int j = 0; j < TP - 1; ++j)

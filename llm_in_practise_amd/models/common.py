@@ -2,6 +2,7 @@
 from __future__ import annotations
 
 import dataclasses
+import functools
 
 import torch
 import torch.nn as nn
@@ -299,11 +300,18 @@ class SeqBatch:
         self.decode = host is None
         self.positions = desc[4][None]
         self.len, self.pos = 0, None                                      # KVCache duck-typing (unused)
-        self.cache_idx = desc[1].long()[desc[3].long()] * cache.max_len + desc[4].long()
-        self.last = (desc[0][1:] - 1).long()
         # a sequence that continues with more than one token: blocks of a kernel that split it over time must not
         # read and write its carried rows in one launch
         self.carried_runs = host is not None and any(p > 0 and b - a > 1 for p, a, b in zip(host[2], host[0], host[0][1:]))
+
+    # (index tensors of the reference ops and of a prefill's callers: built when asked for, a decode step asks for none)
+    @functools.cached_property
+    def cache_idx(self) -> torch.Tensor:
+        return self.desc[1].long()[self.desc[3].long()] * self.cache.max_len + self.desc[4].long()
+
+    @functools.cached_property
+    def last(self) -> torch.Tensor:
+        return (self.desc[0][1:] - 1).long()
 
     @classmethod
     def packed(cls, cache: "SeqStateCache", slots: list[int], lens: list[int], starts: list[int] | None = None):

@@ -829,3 +829,15 @@ def test_decode_graphs_replay_equals_eager():
         close(graph[k], eager[k].double(), 1e-5)
     close(eager["a"], logits_of(cfg, W, a[:29]))
     close(eager["c"], logits_of(cfg, W, c))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("T,K,C", [(1, 1, 1), (3, 12, 130), (8, 16, 64), (9, 128, 200), (64, 256, 65), (65, 40, 70), (5, 300, 33)])
+def test_float_products_of_low_rank(device, T, K, C):
+    """matmul_f32 on column slices of bf16 rows: few and many rows, odd ranks and widths."""
+    from llm_in_practise_amd.ops.gemm import matmul_f32
+    g = torch.Generator().manual_seed(K)
+    wide, w = torch.randn(T, K + 11, generator=g).to(torch.bfloat16), torch.randn(C, K, generator=g).to(torch.bfloat16)
+    got = matmul_f32(wide.to(device)[:, 3:3 + K], w.to(device))
+    assert got.dtype == torch.float32
+    close(got, wide[:, 3:3 + K].double() @ w.double().t(), 1e-5)
