@@ -8,6 +8,20 @@
 
 using namespace lipa;
 
+template <typename T>
+__device__ __forceinline__ f32x4 load4_act(const T* p);
+template <>
+__device__ __forceinline__ f32x4 load4_act<float>(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+template <>
+__device__ __forceinline__ f32x4 load4_act<bf16>(const bf16* p) {
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+__device__ __forceinline__ void store4_act(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+__device__ __forceinline__ void store4_act(bf16* p, f32x4 v) {
+  *reinterpret_cast<bf16x4*>(p) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+}
+
 // x[t, c] = table[tok[t], c] * scale + (c even ? sin : cos)(pos[t] * inv_freq[c / 2])
 template <typename T>
 __global__ __launch_bounds__(256) void k_embed_sincos(const long* __restrict__ tok, const int* __restrict__ pos,
@@ -138,6 +152,35 @@ __global__ __launch_bounds__(256) void k_decay_gate(const float* __restrict__ pr
   g[i] = expf(-expf(a_log[c / dk]) * softplusf_(pre[i] + bias[c]));
 }
 
+// The same with 16-byte accesses: LPR lanes per (token, head) row of dv <= 4 LPR entries, so a lane keeps its four entries
+// between the two passes and a wave serves 64 / LPR rows.
+template <typename T, int LPR>
+__global__ __launch_bounds__(256) void k_head_norm_gate4(const float* __restrict__ o, const float* __restrict__ w,
+                                                         int per_head, const T* __restrict__ gate, int ldg,
+                                                         const float* __restrict__ den, const float* __restrict__ efl,
+                                                         T* __restrict__ out, int ldo, float scale, int nrows, int H,
+                                                         int dv, float eps, int silu) {
+  const int row = blockIdx.x * (256 / LPR) + threadIdx.x / LPR, c = 4 * (threadIdx.x % LPR);
+  const bool on = row < nrows && c < dv;              // (every lane of a row's group takes part in the exchanges)
+  const int t = on ? row / H : 0, hd = on ? row % H : 0;
+  f32x4 v = {0.f, 0.f, 0.f, 0.f}, g = v;
+  if (on) {
+    v = load4_act<float>(o + (size_t)row * dv + c);
+    g = load4_act<T>(gate + (size_t)t * ldg + hd * dv + c);
+    if (den != nullptr) v *= 1.f / (fmaxf(fabsf(den[row]), efl[row]) + 1e-6f);
+  }
+  float s = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+#pragma unroll
+  for (int i = LPR / 2; i > 0; i >>= 1) s += __shfl_xor(s, i, 64);
+  if (!on) return;
+  const float rs = rsqrtf(s / dv + eps) * scale;
+  const f32x4 wv = load4_act<float>(w + (per_head ? hd * dv : 0) + c);
+  f32x4 y;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) y[j] = v[j] * rs * wv[j] * sigmoidf_(g[j]) * (silu ? g[j] : 1.f);
+  store4_act(out + (size_t)t * ldo + hd * dv + c, y);
+}
+
 // x[t] = table[tok[t]] * scale + pair[(prev * mul_prev + tok[t] * mul_cur) mod buckets]; a sequence's first token takes
 // row `buckets`.  prev is the token before: the packed neighbour, or for a step's first token of a continued
 // sequence the slot's carried token.  The block of a sequence's first token of the step also carries the step's last
@@ -205,20 +248,6 @@ __global__ __launch_bounds__(256) void k_rms_act(const T* __restrict__ u, int ld
 // gate first, then norm: v = y * silu(z); out = v / rms_part(v) * w, the row cut into equal parts of `gs` entries.
 // VEC: four columns per thread and step (16-byte loads of y and w, 8- or 16-byte loads of z); the gated values of a
 // thread's first two steps stay in registers for the second pass.
-template <typename T>
-__device__ __forceinline__ f32x4 load4_act(const T* p);
-template <>
-__device__ __forceinline__ f32x4 load4_act<float>(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
-template <>
-__device__ __forceinline__ f32x4 load4_act<bf16>(const bf16* p) {
-  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
-  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
-}
-__device__ __forceinline__ void store4_act(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
-__device__ __forceinline__ void store4_act(bf16* p, f32x4 v) {
-  *reinterpret_cast<bf16x4*>(p) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
-}
-
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void k_gate_group_norm(const float* __restrict__ y, const T* __restrict__ z, int ldz,
                                                          const float* __restrict__ w, T* __restrict__ out, int n, int gs,
@@ -749,6 +778,17 @@ void seq_head_norm_gate(int code, const float* o, const float* w, int per_head, 
                         float eps, int silu, hipStream_t st) {
   const int rows = T_ * H;
   if (rows == 0) return;
+  if (dv % 4 == 0 && dv <= 256 && ldg % 4 == 0 && ldo % 4 == 0 && (((uintptr_t)gate | (uintptr_t)out) & 15) == 0) {
+#define HEAD_NORM4(LPR)                                                                                                   \
+  hipLaunchKernelGGL((k_head_norm_gate4<T, LPR>), dim3((rows + 256 / LPR - 1) / (256 / LPR)), dim3(256), 0, st, o, w, per_head, \
+                     (const T*)gate, ldg, den, efl, (T*)out, ldo, scale, rows, H, dv, eps, silu)
+    SEQ_DISPATCH_T(code, {
+      if (dv <= 32) HEAD_NORM4(8); else if (dv <= 64) HEAD_NORM4(16); else if (dv <= 128) HEAD_NORM4(32); else HEAD_NORM4(64);
+    });
+#undef HEAD_NORM4
+    LIPA_CHECK_LAUNCH();
+    return;
+  }
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_head_norm_gate<T>, dim3((rows + 3) / 4), dim3(256), 0, st, o, w, per_head,
                                           (const T*)gate, ldg, den, efl, (T*)out, ldo, scale, rows, H, dv, eps, silu));
   LIPA_CHECK_LAUNCH();

@@ -681,6 +681,22 @@ def test_bf16_matrix_core_unequal_batch(device):
 
 
 @pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("heads,kv_heads", [(4, 1), (3, 3), (6, 2)])
+@pytest.mark.parametrize("dim", [64, 96, 128])
+def test_bf16_exact_size_sweeps(device, dim, heads, kv_heads):
+    """Head sizes with a sweep of their own (64, 96, 128), with and without bounded scores, in the forms for four heads
+    per kv head, one head and grouped decode heads; 200 tokens cross several whole and cut tiles."""
+    cfg = config([att(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, every=40, scale=0.8 / dim ** 0.5),
+                  par(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, rot=dim // 2, scale=1.2 / dim ** 0.5, cap=2.5, inner=24, state=8,
+                      mlp=ALL)], width=64, mult=0.2)
+    lm, W = build(cfg, device, 33, dtype=torch.bfloat16)
+    toks = tokens(200, cfg["vocab"], 34)
+    want = logits_of(cfg, W, toks)
+    close16(replay(lm, 400, decoding(toks, 185))["a"], want)
+    close16(replay(lm, 400, portions(toks, (33, 64, 2, 101)))["a"], want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
 def test_bf16_wide_heads(device):
     """Heads of 128, 160 and 256 columns (the sweeps' wide instantiations), key size 128 in the linear attention."""
     cfg = config([att(heads=4, kv_heads=1, dim=128, vdim=128, every=30, scale=0.06, mlp=ALL), gla(heads=1, dim=128, vdim=64),
@@ -841,3 +857,23 @@ def test_float_products_of_low_rank(device, T, K, C):
     got = matmul_f32(wide.to(device)[:, 3:3 + K], w.to(device))
     assert got.dtype == torch.float32
     close(got, wide[:, 3:3 + K].double() @ w.double().t(), 1e-5)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dv", [4, 20, 36, 64, 100, 128, 200, 256, 300, 7])
+def test_head_norm_and_gate_read_out(device, dv):
+    """Per-head RMS norm with a shared or per-head weight, sigmoid and SiLU gates, into a scaled column slice."""
+    from llm_in_practise_amd.ops.norm import head_norm_gate
+    g = torch.Generator().manual_seed(dv)
+    T, H = 5, 3
+    o, wide = torch.randn(T, H, dv, generator=g), torch.randn(T, H * dv + 8, generator=g)
+    gate = wide[:, 8:]
+    for act, w in (("sigmoid", torch.randn(dv, generator=g)), ("silu", torch.randn(H * dv, generator=g))):
+        z = gate.double()
+        want = O.unit_rms(o.double(), 1e-5) * (w.double() if w.numel() == dv else w.double().view(H, dv))
+        want = want.reshape(T, -1) * (torch.sigmoid(z) if act == "sigmoid" else O.silu(z))
+        close(head_norm_gate(o.to(device), w.to(device), wide.to(device)[:, 8:], 1e-5, act=act), want, 1e-5)
+        out = torch.zeros(T, H * dv + 4, device=device)
+        head_norm_gate(o.to(device), w.to(device), wide.to(device)[:, 8:], 1e-5, out=out[:, 4:], scale=-0.3, act=act)
+        close(out[:, 4:], -0.3 * want, 1e-5)
+        assert bool((out[:, :4] == 0).all())
