@@ -13,8 +13,8 @@
 // head, and three optional parts change which keys count and how: a float bias per (head, distance) added to the
 // scaled score, a block mask (a query sees only the keys of its own run of `block` positions, counted from the
 // sequence's position 0), a sliding window (a query sees only the keys less than `window` positions back, itself
-// included), and a sink (one more key of a fixed score, or of a learned score per head, without a value in every
-// softmax).  With one key split the matrix-core sweep normalises and writes the activation type itself; otherwise
+// included; the sequence's first `keep` keys may stay visible behind it), and a sink (one more key of a fixed score, or
+// of a learned score per head, without a value in every softmax).  With one key split the matrix-core sweep normalises and writes the activation type itself; otherwise
 // k_gqa_merge does.  Scores may be bounded (softcap * tanh(score / softcap)), the result may be multiplied element by
 // element with the sigmoid of a gate.  The output may be a column slice of a wider matrix (row stride ldo) and is multiplied by
 // out_scale.
@@ -37,6 +37,7 @@ struct GqaExtra {
   float softcap;       // 0: plain scores
   const void* gate;    // [T, H * dv] gate pre-activations in the activation type or null; rows ldg apart (8-byte rows)
   int ldg;
+  int keep;            // with a window: keys j < keep are seen from any distance
 };
 
 constexpr int MAXC = 16;   // value columns per lane: G * dv <= 64 * MAXC
@@ -55,8 +56,12 @@ __global__ __launch_bounds__(64) void k_talk_attn_partial(const T* __restrict__ 
   __syncthreads();
   int lo = (GQA && x.block > 0) ? (p / x.block) * x.block : 0;
   if (GQA && x.window > 0) lo = max(lo, p - x.window + 1);
-  const int nkeys = p + 1 - lo, per = (nkeys + nsplit - 1) / nsplit;
-  const int j0 = lo + z * per, j1 = min(p + 1, j0 + per);
+  // the sweep's index runs over the kept keys that lie before the window, then over the window: base .. lo - 1 stand for
+  // keys 0 .. lo - base - 1, and from lo on an index is its key
+  const int base = lo - ((GQA && x.window > 0) ? min(x.keep, lo) : 0);
+  const int nkeys = p + 1 - base, per = (nkeys + nsplit - 1) / nsplit;
+  const int j0 = base + z * per, j1 = min(p + 1, j0 + per);
+  auto key_of = [&](int j) { return j < lo ? j - base : j; };
   const T* kbase = kc + ((size_t)slot * max_len) * ldk + kh * dk;
   const T* vbase = vc + ((size_t)slot * max_len) * ldv + (GQA ? kh * dv : 0);
   float acc[MAXC];
@@ -67,12 +72,12 @@ __global__ __launch_bounds__(64) void k_talk_attn_partial(const T* __restrict__ 
     const int j = jb + lane;
     float sc = -INFINITY;
     if (j < j1) {
-      const T* kr = kbase + (size_t)j * ldk;
+      const T* kr = kbase + (size_t)key_of(j) * ldk;
       float a = 0.f;
       for (int i = 0; i < dk; ++i) a += sq[i] * (float)kr[i];
       sc = a * scale;
       if (GQA && x.softcap > 0.f) sc = x.softcap * tanhf(sc / x.softcap);
-      if (GQA && x.bias != nullptr) sc += x.bias[(size_t)g * x.nd + min(p - j, x.nd - 1)];
+      if (GQA && x.bias != nullptr) sc += x.bias[(size_t)g * x.nd + min(p - key_of(j), x.nd - 1)];
     }
     const float mn = fmaxf(m, wave_max(sc));
     if (mn == -INFINITY) continue;            // a split without keys (lanes agree: mn is wave-uniform)
@@ -85,7 +90,7 @@ __global__ __launch_bounds__(64) void k_talk_attn_partial(const T* __restrict__ 
     const int cnt = min(64, j1 - jb);
     for (int jj = 0; jj < cnt; ++jj) {
       const float wj = __shfl(w, jj, 64);
-      const T* vr = vbase + (size_t)(jb + jj) * ldv;
+      const T* vr = vbase + (size_t)key_of(jb + jj) * ldv;
 #pragma unroll
       for (int c = 0; c < MAXC; ++c) {
         const int col = c * 64 + lane;
@@ -157,6 +162,11 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
     lo_t = max(lo_t, (HEADS ? pos_q : d.tok_pos[t0]) - win + 1);
     lo_q = max(lo_q, pos_q - win + 1);
   }
+  // kept first keys: the sweep's index runs over those before the window, then over the window (base .. lo_t - 1 stand for
+  // keys 0 .. lo_t - base - 1, and from lo_t on an index is its key)
+  const int keep = (GQA && win > 0) ? x.keep : 0, base = lo_t - min(keep, lo_t);
+  auto key_of = [&](int j) { return j < lo_t ? j - base : j; };
+  auto row_of = [&](int j) { return (size_t)min(key_of(j), max_len - 1); };
   const float* brow = (!EXACT && GQA && x.bias != nullptr) ? x.bias + (size_t)g * x.nd : nullptr;
   // a tile's queries sit at consecutive positions p0 + ql, so a 32-key tile meets only the 63 distances
   // p0 - jb - 31 + i: lane i fetches that one bias and the 16 a lane needs come from its neighbours' registers
@@ -168,7 +178,7 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
   // from this key on every query of the tile sees a key that is not in its future
   const int lo_all = EXACT ? (blk > 0 ? (pmax / blk) * blk : win > 0 ? pmax - win + 1 : 0) : 0;
   const int trow = 4 * (lane >> 5) + ((lane & 15) >> 2), tcol = 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
-  const int per = (pmax - lo_t + nsplit) / nsplit, j0 = lo_t + z * per, j1 = min(pmax + 1, j0 + per);
+  const int per = (pmax - base + nsplit) / nsplit, j0 = base + z * per, j1 = min(pmax + 1, j0 + per);
   const bf16* kbase = kc + ((size_t)slot * max_len) * ldk + kh * dk + 8 * hi;
   const bf16* vbase = vc + ((size_t)slot * max_len) * ldv + c * dv;
   bf16x8 qf[NDS];
@@ -192,19 +202,19 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
     for (int i = 0; i < VPT; ++i) {
       const int e = threadIdx.x + 64 * NW * i, row = e / vpr, cv = e % vpr;
       if ((EXACT && (2 * NDT) % NW == 0) || e < 32 * vpr)
-        pv[i] = *reinterpret_cast<const bf16x8*>(vbase + (size_t)min(jb + row, max_len - 1) * ldv + cv * 8);
+        pv[i] = *reinterpret_cast<const bf16x8*>(vbase + row_of(jb + row) * ldv + cv * 8);
     }
     if (NW == 1) {
 #pragma unroll
       for (int i = 0; i < KPT; ++i)
-        pk[i] = *reinterpret_cast<const bf16x8*>(kbase + (size_t)min(jb + ql, max_len - 1) * ldk + 16 * i);
+        pk[i] = *reinterpret_cast<const bf16x8*>(kbase + row_of(jb + ql) * ldk + 16 * i);
       return;
     }
 #pragma unroll
     for (int i = 0; i < KPT; ++i) {
       const int e = threadIdx.x + 64 * NW * i, row = e / kpr, cv = e % kpr;
       if ((EXACT && NDS % NW == 0) || e < 32 * kpr)
-        pk[i] = *reinterpret_cast<const bf16x8*>(kbase - 8 * hi + (size_t)min(jb + row, max_len - 1) * ldk + cv * 8);
+        pk[i] = *reinterpret_cast<const bf16x8*>(kbase - 8 * hi + row_of(jb + row) * ldk + cv * 8);
     }
   };
   if (AHEAD && j0 < j1) fetch(j0);
@@ -221,7 +231,7 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
       for (int e = threadIdx.x; e < 32 * vpr; e += 64) {
         const int row = e / vpr, cv = e % vpr;
         *reinterpret_cast<bf16x8*>(sV + row * LD + cv * 8) =
-            *reinterpret_cast<const bf16x8*>(vbase + (size_t)min(jb + row, max_len - 1) * ldv + cv * 8);
+            *reinterpret_cast<const bf16x8*>(vbase + row_of(jb + row) * ldv + cv * 8);
       }
     }
     if (NW > 1) {
@@ -242,7 +252,7 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
       for (int ds = 0; ds < NDS; ++ds) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pk[ds < KPT ? ds : 0], qf[ds], sc, 0, 0, 0);
       if (jb + 32 < j1) fetch(jb + 32);
     } else {
-      const bf16* kr = NW > 1 ? sK + ql * LDK + 8 * hi : kbase + (size_t)min(jb + ql, max_len - 1) * ldk;
+      const bf16* kr = NW > 1 ? sK + ql * LDK + 8 * hi : kbase + row_of(jb + ql) * ldk;
 #pragma unroll
       for (int ds = 0; ds < NDS; ++ds)
         if (EXACT || ds < nds)
@@ -254,7 +264,7 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
     auto score = [&](float a) {
       return capped ? cl2 - 2.f * cl2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(a * ce) + 1.f) : a * sl2;
     };
-    if (EXACT && jb + 31 <= p0 && jb + 32 <= j1 && jb >= lo_all) {      // every query sees the whole tile
+    if (EXACT && jb + 31 <= p0 && jb + 32 <= j1 && (jb >= lo_all || jb + 32 <= lo_t)) {      // every query sees the whole tile
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         sc[r] = score(sc[r]);
@@ -263,8 +273,8 @@ __global__ __launch_bounds__(64 * NW, EXACT ? 2 : 1) void k_talk_attn_mfma(const
     } else {
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
-        const int kk = (r & 3) + 8 * (r >> 2) + 4 * hi, key = jb + kk;
-        const bool seen = key <= pos_q && key < j1 && (!GQA || key >= lo_q);
+        const int kk = (r & 3) + 8 * (r >> 2) + 4 * hi, key = key_of(jb + kk);
+        const bool seen = key <= pos_q && jb + kk < j1 && (!GQA || key >= lo_q || key < keep);
         float v = score(sc[r]);
         if (!EXACT && GQA && !HEADS && brow != nullptr) v += __shfl(bw, ql - kk + 31, 64);
         if (!EXACT && GQA && HEADS && brow != nullptr && seen) v += brow[min(pos_q - key, x.nd - 1)] * 1.4426950408889634f;
@@ -463,7 +473,7 @@ void seq_attn_sweep(int code, const void* q, int ldq, const void* kc, int ldk, c
                     float* pl, float* pu, int H, int G, int dk, int dv, int max_len, int nsplit, float scale,
                     const int* tile_seq, const int* tile_t0, int ntiles, SeqDesc d, hipStream_t st) {
   sweep<false>(code, q, ldq, kc, ldk, vc, ldv, pm, pl, pu, H, G, dk, dv, max_len, nsplit, scale, tile_seq, tile_t0,
-               ntiles, d, GqaExtra{nullptr, 0, 0, 0, 0.f, nullptr, 0, nullptr, 0, 1.f, 0.f, nullptr, 0}, st);
+               ntiles, d, GqaExtra{nullptr, 0, 0, 0, 0.f, nullptr, 0, nullptr, 0, 1.f, 0.f, nullptr, 0, 0}, st);
 }
 
 // Merge of a GQA sweep's key splits: one block of four waves per (token, head), a wave takes every fourth split, so the
@@ -510,19 +520,19 @@ __global__ __launch_bounds__(256) void k_gqa_merge(const float* __restrict__ pm,
   }
 }
 
-// Grouped-query attention over a slot-indexed cache with an optional distance bias, block mask, sliding window and
-// sink.  Key rows are ldk and value rows ldv elements apart (values may be columns of the key rows: a latent cache
+// Grouped-query attention over a slot-indexed cache with an optional distance bias, block mask, sliding window (behind
+// which the first `keep` keys may stay visible; not with a bias) and sink.  Key rows are ldk and value rows ldv elements apart (values may be columns of the key rows: a latent cache
 // with G = 1); the output rows are ldo elements apart.
 void seq_gqa_attention(int code, const void* q, int ldq, const void* kc, int ldk, const void* vc, int ldv, float* pm,
                        float* pl, float* pu, const float* bias, int nd, int block, int window, int sink, float sink_logit,
                        const float* sinks, void* out, int ldo, float out_scale, float softcap, const void* gate, int ldg,
-                       int H, int G, int dk, int dv, int max_len, int nsplit, float scale, const int* tile_seq,
+                       int keep, int H, int G, int dk, int dv, int max_len, int nsplit, float scale, const int* tile_seq,
                        const int* tile_t0, int ntiles, SeqDesc d, hipStream_t st) {
   if (d.Ttot == 0) return;
   const bool direct = sweep<true>(code, q, ldq, kc, ldk, vc, ldv, pm, pl, pu, H, G, dk, dv, max_len, nsplit, scale,
                                   tile_seq, tile_t0, ntiles, d,
                                   GqaExtra{bias, nd, block, sink, sink_logit, out, window, sinks, ldo, out_scale, softcap,
-                                           gate, ldg}, st);
+                                           gate, ldg, keep}, st);
   if (direct) return;
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_gqa_merge<T>, dim3(d.Ttot, H), dim3(256), 0, st, pm, pl, pu, (T*)out, H, dv,
                                           nsplit, sink, sink_logit, sinks, ldo, out_scale, (const T*)gate, ldg));

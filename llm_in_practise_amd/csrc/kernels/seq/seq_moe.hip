@@ -2,7 +2,8 @@
 // correction and identity experts; a few-token path in which every (token, chosen expert) pair streams its expert's
 // rows (no sort, no host round trip: decode steps and hipGraphs); and the weighted combine of expert outputs.
 // Routing variants (`kind` bits): scores as each output's own sigmoid instead of the softmax (1), a group ranked by the
-// sum of its two largest choices instead of its largest (2), weights divided by their sum over the chosen (4).
+// sum of its two largest choices instead of its largest (2), weights divided by their sum over the chosen (4), the
+// correction added to the logits, so that it moves the scores and weights too (8).
 // Experts are clipped GLUs or SiLU GLUs; a pair's weight multiplies the expert's output or its input; the shared expert may sit behind a per-token sigmoid gate.
 // Router scores, weights and the combine are float; expert products read the activation type and accumulate in float.
 #include "seq_common.h"
@@ -38,6 +39,7 @@ __device__ __forceinline__ void route_wave(const float* z, const float* __restri
     const int e = lane + 64 * i;
     // a row nobody reads (an idle decode row) may carry anything, NaN included: it still gets ids inside [0, n)
     s[i] = e < n ? (isfinite(z[e]) ? z[e] : 0.f) : -INFINITY;
+    if ((kind & 8) && e < n && corr != nullptr) s[i] += corr[e];
     mx = fmaxf(mx, s[i]);
   }
   mx = wave_max(mx);
@@ -55,7 +57,7 @@ __device__ __forceinline__ void route_wave(const float* z, const float* __restri
   for (int i = 0; i < RPL; ++i) {
     const int e = lane + 64 * i;
     s[i] /= sum;
-    ch[i] = e < n ? s[i] + (corr != nullptr ? corr[e] : 0.f) : -INFINITY;
+    ch[i] = e < n ? s[i] + (corr != nullptr && !(kind & 8) ? corr[e] : 0.f) : -INFINITY;
   }
   if (groups > 1 && keep < groups && (kind & 2)) {
     // rank of group g = its largest choice + its second largest (a group of one: the one), held by lane g

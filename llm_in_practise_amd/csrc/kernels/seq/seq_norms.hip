@@ -230,6 +230,77 @@ __global__ __launch_bounds__(256) void k_scaled_postnorm(float* __restrict__ x, 
   }
 }
 
+// The exit of a sublayer whose OUTPUT is normed: x <- x + rms(y) * w in place (float), h = x in the activation type or,
+// with wn (the model's last norm), rms(x) * wn.  VEC: four columns per thread and step with 16-byte accesses; a thread
+// keeps its first four steps (widths up to 4096) in registers between the passes.
+template <typename T, typename YT, bool VEC>
+__global__ __launch_bounds__(256) void k_residual_postnorm(float* __restrict__ x, const YT* __restrict__ y, int ldy,
+                                                           const float* __restrict__ w, const float* __restrict__ wn,
+                                                           T* __restrict__ h, int W, float eps) {
+  __shared__ float sc[4];
+  const size_t t = blockIdx.x;
+  float* xr = x + t * W;
+  const YT* yr = y + t * ldy;
+  T* hr = h + t * W;
+  float s = 0.f, s2 = 0.f;
+  if (VEC) {
+    constexpr int KEEP = 4;
+    f32x4 ky[KEEP], kx[KEEP];
+    auto sq = [](f32x4 v) { return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; };
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int c = 4 * threadIdx.x + 1024 * i;
+      if (c < W) {
+        ky[i] = load4_act<YT>(yr + c);
+        kx[i] = load4_act<float>(xr + c);
+        s += sq(ky[i]);
+      }
+    }
+    for (int c = 4 * threadIdx.x + 1024 * KEEP; c < W; c += 1024) s += sq(load4_act<YT>(yr + c));
+    const float rs = rsqrtf(block_sum256(s, sc) / W + eps);
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int c = 4 * threadIdx.x + 1024 * i;
+      if (c < W) {
+        kx[i] += ky[i] * load4_act<float>(w + c) * rs;
+        store4_act(xr + c, kx[i]);
+        if (wn == nullptr) store4_act(hr + c, kx[i]);
+        s2 += sq(kx[i]);
+      }
+    }
+    for (int c = 4 * threadIdx.x + 1024 * KEEP; c < W; c += 1024) {
+      const f32x4 v = load4_act<float>(xr + c) + load4_act<YT>(yr + c) * load4_act<float>(w + c) * rs;
+      store4_act(xr + c, v);
+      if (wn == nullptr) store4_act(hr + c, v);
+      s2 += sq(v);
+    }
+    if (wn == nullptr) return;
+    const float rs2 = rsqrtf(block_sum256(s2, sc) / W + eps);
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int c = 4 * threadIdx.x + 1024 * i;
+      if (c < W) store4_act(hr + c, kx[i] * load4_act<float>(wn + c) * rs2);
+    }
+    for (int c = 4 * threadIdx.x + 1024 * KEEP; c < W; c += 1024)      // the thread re-reads the columns it wrote itself
+      store4_act(hr + c, load4_act<float>(xr + c) * load4_act<float>(wn + c) * rs2);
+    return;
+  }
+  for (int c = threadIdx.x; c < W; c += 256) {
+    const float v = (float)yr[c];
+    s += v * v;
+  }
+  const float rs = rsqrtf(block_sum256(s, sc) / W + eps);
+  for (int c = threadIdx.x; c < W; c += 256) {
+    const float v = xr[c] + (float)yr[c] * rs * w[c];
+    xr[c] = v;
+    if (wn == nullptr) hr[c] = (T)v;
+    s2 += v * v;
+  }
+  if (wn == nullptr) return;
+  const float rs2 = rsqrtf(block_sum256(s2, sc) / W + eps);
+  for (int c = threadIdx.x; c < W; c += 256) hr[c] = (T)(xr[c] * rs2 * wn[c]);
+}
+
 // RMS norm of activation rows (a column slice of a wider matrix is fine)
 template <typename T>
 __global__ __launch_bounds__(256) void k_rms_act(const T* __restrict__ u, int ldu, const float* __restrict__ w,
@@ -497,17 +568,63 @@ __global__ __launch_bounds__(256) void k_qk_norm_store(const T* __restrict__ u, 
   }
 }
 
+// A token's value row on its way into the cache (256 threads): as it comes, every head (dv entries) over its root mean
+// square (veps >= 0; one wave per head), or blended with the row `first` of another cache, (1 - lam) v + lam first.
+template <typename T>
+__device__ __forceinline__ void store_values(const T* __restrict__ vr, T* __restrict__ dst, const T* __restrict__ first,
+                                             float lam, int nv, int dv, float veps) {
+  if (veps >= 0.f) {
+    const int lane = threadIdx.x & 63;
+    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
+      float ss = 0.f;
+      for (int c = lane; c < dv; c += 64) {
+        const float v = (float)vr[h0 + c];
+        ss += v * v;
+      }
+      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
+      for (int c = lane; c < dv; c += 64) dst[h0 + c] = (T)((float)vr[h0 + c] * rs);
+    }
+  } else if (first != nullptr) {
+    for (int c = threadIdx.x; c < nv; c += 256) dst[c] = (T)((1.f - lam) * (float)vr[c] + lam * (float)first[c]);
+  } else {
+    for (int c = threadIdx.x; c < nv; c += 256) dst[c] = vr[c];
+  }
+}
+
+// The same, four entries per thread (dv a multiple of 4, 16-byte or 8-byte rows).
+template <typename T>
+__device__ __forceinline__ void store_values4(const T* __restrict__ vr, T* __restrict__ dst, const T* __restrict__ first,
+                                              float lam, int nv, int dv, float veps) {
+  if (veps >= 0.f) {
+    const int lane = threadIdx.x & 63;
+    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
+      float ss = 0.f;
+      for (int c = 4 * lane; c < dv; c += 256) {
+        const f32x4 v = load4_act<T>(vr + h0 + c);
+        ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+      }
+      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
+      for (int c = 4 * lane; c < dv; c += 256) store4_act(dst + h0 + c, load4_act<T>(vr + h0 + c) * rs);
+    }
+  } else if (first != nullptr) {
+    for (int c = 4 * threadIdx.x; c < nv; c += 1024)
+      store4_act(dst + c, load4_act<T>(vr + c) * (1.f - lam) + load4_act<T>(first + c) * lam);
+  } else {
+    for (int c = 4 * threadIdx.x; c < nv; c += 1024) store4_act(dst + c, load4_act<T>(vr + c));
+  }
+}
+
 // A step's [q | k (| v)] rows on their way into rotary attention: the first `dims` entries of every q and k head are
 // rotated at the token's position; the rotated k goes to the key cache; the value cache gets the v columns or, with
 // vkeys, the k columns as they came (a design whose values are its unrotated keys).  tevery > 0: q is multiplied by
 // 1 + tcoef ln(floor((pos + 1) / tevery) + 1).  veps >= 0: every head's value (dv entries) is divided by its root mean
-// square.  One block per token.
+// square.  vfirst: the values are blended with another cache's row of the same slot and position.  One block per token.
 template <typename T>
 __global__ __launch_bounds__(256) void k_rope_kv_store(const T* __restrict__ u, int ldu, const float* __restrict__ inv_freq,
                                                        T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
                                                        int nq, int nk, int nv, int dk, int dims, int half, float mag,
                                                        int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
-                                                       SeqDesc d) {
+                                                       const T* __restrict__ vfirst, float lam, SeqDesc d) {
   const size_t t = blockIdx.x;
   const T* r = u + t * ldu;
   const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]];
@@ -524,20 +641,8 @@ __global__ __launch_bounds__(256) void k_rope_kv_store(const T* __restrict__ u, 
     kc[row * nk + c] = (T)rotated_at(r + nq + (c - cl), cl, dims, p, inv_freq, half, mag);
     if (vkeys && veps < 0.f) vc[row * nk + c] = r[nq + c];
   }
-  if (veps >= 0.f) {                                 // one wave per head: the value over its root mean square
-    const T* vr = r + (vkeys ? nq : nq + nk);
-    const int lane = threadIdx.x & 63;
-    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
-      float ss = 0.f;
-      for (int c = lane; c < dv; c += 64) {
-        const float v = (float)vr[h0 + c];
-        ss += v * v;
-      }
-      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
-      for (int c = lane; c < dv; c += 64) vc[row * nv + h0 + c] = (T)((float)vr[h0 + c] * rs);
-    }
-  } else if (!vkeys)
-    for (int c = threadIdx.x; c < nv; c += 256) vc[row * nv + c] = r[nq + nk + c];
+  if (veps >= 0.f || !vkeys)
+    store_values<T>(r + (vkeys ? nq : nq + nk), vc + row * nv, vfirst != nullptr ? vfirst + row * nv : nullptr, lam, nv, dv, veps);
 }
 
 // The same, four entries per thread (16-byte or 8-byte accesses; dk and dv multiples of 4, dims of 8 when `half`).
@@ -546,7 +651,7 @@ __global__ __launch_bounds__(256) void k_rope_kv_store4(const T* __restrict__ u,
                                                         T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
                                                         int nq, int nk, int nv, int dk, int dims, int half, float mag,
                                                         int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
-                                                        SeqDesc d) {
+                                                        const T* __restrict__ vfirst, float lam, SeqDesc d) {
   const size_t t = blockIdx.x;
   const T* r = u + t * ldu;
   const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]], hd = dims >> 1;
@@ -589,20 +694,117 @@ __global__ __launch_bounds__(256) void k_rope_kv_store4(const T* __restrict__ u,
     }
   }
   if (!keep) return;
-  const T* vr = r + (vkeys ? nq : nq + nk);
-  if (veps >= 0.f) {                                 // one wave per head: the value over its root mean square
-    const int lane = threadIdx.x & 63;
-    for (int h0 = (threadIdx.x >> 6) * dv; h0 < nv; h0 += 4 * dv) {
-      float ss = 0.f;
-      for (int c = 4 * lane; c < dv; c += 256) {
-        const f32x4 v = load4_act<T>(vr + h0 + c);
-        ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-      }
-      const float rs = rsqrtf(wave_sum(ss) / dv + veps);
-      for (int c = 4 * lane; c < dv; c += 256) store4_act(vc + row * nv + h0 + c, load4_act<T>(vr + h0 + c) * rs);
+  if (veps >= 0.f || !vkeys)
+    store_values4<T>(r + (vkeys ? nq : nq + nk), vc + row * nv, vfirst != nullptr ? vfirst + row * nv : nullptr, lam, nv, dv, veps);
+}
+
+// The same with a norm: every q and k head is rotated, then divided by its root mean square (qkeps inside the root).  One
+// block per token; its sines and cosines are taken once, into LDS, and serve all heads.  One wave per head.
+template <typename T>
+__global__ __launch_bounds__(256) void k_rope_norm_store(const T* __restrict__ u, int ldu, const float* __restrict__ inv_freq,
+                                                         T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
+                                                         int nq, int nk, int nv, int dk, int dims, int half, float mag,
+                                                         int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
+                                                         float qkeps, const T* __restrict__ vfirst, float lam, SeqDesc d) {
+  extern __shared__ float scs[];                     // [dims / 2] sines, [dims / 2] cosines
+  const size_t t = blockIdx.x;
+  const T* r = u + t * ldu;
+  const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]], hd = dims >> 1, lane = threadIdx.x & 63;
+  for (int i = threadIdx.x; i < hd; i += 256) {
+    float sn, cs;
+    sincosf((float)pos * inv_freq[i], &sn, &cs);
+    scs[i] = sn * mag;
+    scs[hd + i] = cs * mag;
+  }
+  __syncthreads();
+  const float temp = tevery > 0 && pos >= 0 ? 1.f + tcoef * logf((float)((pos + 1) / tevery + 1)) : 1.f;
+  const bool keep = pos >= 0 && pos < max_len;       // a row nobody reads may carry any position
+  const size_t row = (size_t)slot * max_len + (keep ? pos : 0);
+  for (int c0 = (threadIdx.x >> 6) * dk; c0 < nq + nk; c0 += 4 * dk) {
+    const bool isq = c0 < nq;
+    if (!isq && !keep) break;
+    auto rotated = [&](int c) {
+      const float a = (float)r[c0 + c];
+      if (c >= dims) return a;
+      const bool second = half ? c >= hd : (c & 1);
+      const int pair = half ? (second ? c - hd : c) : (c >> 1);
+      const float b = (float)r[c0 + (half ? (second ? c - hd : c + hd) : (c ^ 1))];
+      return second ? a * scs[hd + pair] + b * scs[pair] : a * scs[hd + pair] - b * scs[pair];
+    };
+    float ss = 0.f;
+    for (int c = lane; c < dk; c += 64) {
+      const float v = rotated(c);
+      ss += v * v;
     }
-  } else if (!vkeys)
-    for (int c = 4 * threadIdx.x; c < nv; c += 1024) store4_act(vc + row * nv + c, load4_act<T>(vr + c));
+    const float rs = rsqrtf(wave_sum(ss) / dk + qkeps) * (isq ? temp : 1.f);
+    T* dst = isq ? qout + t * nq + c0 : kc + row * nk + c0 - nq;
+    for (int c = lane; c < dk; c += 64) dst[c] = (T)(rotated(c) * rs);
+  }
+  if (keep)
+    store_values<T>(r + (vkeys ? nq : nq + nk), vc + row * nv, vfirst != nullptr ? vfirst + row * nv : nullptr, lam, nv, dv, veps);
+}
+
+// The same, four entries per lane: LPR lanes hold a head of dk <= 4 LPR entries between its norm's sum and its store, a
+// block of 256 threads takes 256 / LPR heads at a time (alignments as in k_rope_kv_store4).
+template <typename T, int LPR>
+__global__ __launch_bounds__(256) void k_rope_norm_store4(const T* __restrict__ u, int ldu, const float* __restrict__ inv_freq,
+                                                          T* __restrict__ qout, T* __restrict__ kc, T* __restrict__ vc,
+                                                          int nq, int nk, int nv, int dk, int dims, int half, float mag,
+                                                          int vkeys, int max_len, float tcoef, int tevery, float veps, int dv,
+                                                          float qkeps, const T* __restrict__ vfirst, float lam, SeqDesc d) {
+  extern __shared__ float scs[];
+  const size_t t = blockIdx.x;
+  const T* r = u + t * ldu;
+  const int pos = d.tok_pos[t], slot = d.slots[d.tok_seq[t]], hd = dims >> 1;
+  for (int i = threadIdx.x; i < hd; i += 256) {
+    float sn, cs;
+    sincosf((float)pos * inv_freq[i], &sn, &cs);
+    scs[i] = sn * mag;
+    scs[hd + i] = cs * mag;
+  }
+  __syncthreads();
+  const float temp = tevery > 0 && pos >= 0 ? 1.f + tcoef * logf((float)((pos + 1) / tevery + 1)) : 1.f;
+  const bool keep = pos >= 0 && pos < max_len;       // a row nobody reads may carry any position
+  const size_t row = (size_t)slot * max_len + (keep ? pos : 0);
+  const int c = 4 * (threadIdx.x % LPR);
+  for (int g0 = 0; g0 < nq + nk; g0 += 256 / LPR * dk) {      // (every lane takes part in the exchanges)
+    const int c0 = g0 + (int)(threadIdx.x / LPR) * dk;
+    const bool isq = c0 < nq, on = c0 < nq + nk && c < dk && (isq || keep);
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    if (on) {
+      const f32x4 a = load4_act<T>(r + c0 + c);
+      o = a;
+      if (c < dims) {
+        if (half) {
+          const bool second = c >= hd;
+          const int pair = second ? c - hd : c;
+          const f32x4 b = load4_act<T>(r + c0 + (second ? c - hd : c + hd));
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const float sn = scs[pair + j], cs = scs[hd + pair + j];
+            o[j] = second ? a[j] * cs + b[j] * sn : a[j] * cs - b[j] * sn;
+          }
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; j += 2)
+            if (c + j < dims) {
+              const float sn = scs[(c + j) >> 1], cs = scs[hd + ((c + j) >> 1)];
+              o[j] = a[j] * cs - a[j + 1] * sn;
+              o[j + 1] = a[j + 1] * cs + a[j] * sn;
+            }
+        }
+      }
+    }
+    float ss = o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
+#pragma unroll
+    for (int i = LPR / 2; i > 0; i >>= 1) ss += __shfl_xor(ss, i, 64);
+    if (on) {
+      const float rs = rsqrtf(ss / dk + qkeps) * (isq ? temp : 1.f);
+      store4_act(isq ? qout + t * nq + c0 + c : kc + row * nk + c0 - nq + c, o * rs);
+    }
+  }
+  if (keep)
+    store_values4<T>(r + (vkeys ? nq : nq + nk), vc + row * nv, vfirst != nullptr ? vfirst + row * nv : nullptr, lam, nv, dv, veps);
 }
 
 // out = y * sigmoid(gate), element by element; gate rows are ldg apart
@@ -690,19 +892,26 @@ __global__ __launch_bounds__(256) void k_delta_gates(const T* __restrict__ k, in
 
 void seq_rope_kv_store(int code, const void* u, int ldu, const float* inv_freq, void* qout, void* kc, void* vc, int nq,
                        int nk, int nv, int dk, int dims, int half, float mag, int vkeys, int max_len, float tcoef,
-                       int tevery, float veps, int dv, SeqDesc d, hipStream_t st) {
+                       int tevery, float veps, int dv, float qkeps, const void* vfirst, float lam, SeqDesc d,
+                       hipStream_t st) {
   if (d.Ttot == 0) return;
   const bool vec = ldu % 4 == 0 && dk % 4 == 0 && dv % 4 == 0 && (!half || dims % 8 == 0) && ((uintptr_t)u & 15) == 0;
-  if (vec) {
-    SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_rope_kv_store4<T>, dim3(d.Ttot), dim3(256), 0, st, (const T*)u, ldu, inv_freq,
-                                            (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef,
-                                            tevery, veps, dv, d));
-    LIPA_CHECK_LAUNCH();
-    return;
+#define ROPE_STORE(KERNEL, LDS, ...)                                                                                     \
+  SEQ_DISPATCH_T(code, hipLaunchKernelGGL(KERNEL, dim3(d.Ttot), dim3(256), LDS, st, (const T*)u, ldu, inv_freq, (T*)qout, \
+                                          (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef, tevery, \
+                                          veps, dv, __VA_ARGS__ (const T*)vfirst, lam, d))
+  const size_t lds = sizeof(float) * dims;
+  if (qkeps < 0.f) {
+    if (vec) ROPE_STORE(k_rope_kv_store4<T>, 0, ); else ROPE_STORE(k_rope_kv_store<T>, 0, );
+  } else if (vec && dk <= 256) {
+    if (dk <= 32) ROPE_STORE((k_rope_norm_store4<T, 8>), lds, qkeps,);
+    else if (dk <= 64) ROPE_STORE((k_rope_norm_store4<T, 16>), lds, qkeps,);
+    else if (dk <= 128) ROPE_STORE((k_rope_norm_store4<T, 32>), lds, qkeps,);
+    else ROPE_STORE((k_rope_norm_store4<T, 64>), lds, qkeps,);
+  } else {
+    ROPE_STORE(k_rope_norm_store<T>, lds, qkeps,);
   }
-  SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_rope_kv_store<T>, dim3(d.Ttot), dim3(256), 0, st, (const T*)u, ldu, inv_freq,
-                                          (T*)qout, (T*)kc, (T*)vc, nq, nk, nv, dk, dims, half, mag, vkeys, max_len, tcoef,
-                                          tevery, veps, dv, d));
+#undef ROPE_STORE
   LIPA_CHECK_LAUNCH();
 }
 
@@ -821,6 +1030,23 @@ void seq_scaled_postnorm(int code, int y_f32, float* x, const void* y, int ldy, 
       hipLaunchKernelGGL((k_scaled_postnorm<T, T>), dim3(T_), dim3(256), 0, st, x, (const T*)y, ldy, w, (T*)h, W, alpha,
                          eps);
   });
+  LIPA_CHECK_LAUNCH();
+}
+
+void seq_residual_postnorm(int code, int y_f32, float* x, const void* y, int ldy, const float* w, const float* wn, void* h,
+                           int T_, int W, float eps, hipStream_t st) {
+  if (T_ == 0) return;
+  const bool vec = W % 4 == 0 && ldy % 4 == 0 && ((uintptr_t)y & 15) == 0;      // 16-byte rows (x, w, h are whole tensors)
+#define POSTNORM(YT, VEC)                                                                                            \
+  hipLaunchKernelGGL((k_residual_postnorm<T, YT, VEC>), dim3(T_), dim3(256), 0, st, x, (const YT*)y, ldy, w, wn, (T*)h, W, eps)
+  SEQ_DISPATCH_T(code, {
+    if (y_f32) {
+      if (vec) POSTNORM(float, true); else POSTNORM(float, false);
+    } else {
+      if (vec) POSTNORM(T, true); else POSTNORM(T, false);
+    }
+  });
+#undef POSTNORM
   LIPA_CHECK_LAUNCH();
 }
 

@@ -36,6 +36,7 @@ void seq_ssd_scan(int, const void*, int, const void*, int, const void*, int, con
 void seq_embed_pair(int, const long*, const void*, const void*, int*, float*, void*, int, float, long, long, long,
                     SeqDesc, hipStream_t);
 void seq_scaled_postnorm(int, int, float*, const void*, int, const float*, void*, int, int, float, float, hipStream_t);
+void seq_residual_postnorm(int, int, float*, const void*, int, const float*, const float*, void*, int, int, float, hipStream_t);
 void seq_rms_act(int, const void*, int, const float*, void*, int, int, float, hipStream_t);
 void seq_gate_group_norm(int, const float*, const void*, int, const float*, void*, int, int, int, float, hipStream_t);
 void seq_attn_sweep(int, const void*, int, const void*, int, const void*, int, float*, float*, float*, int, int, int,
@@ -61,9 +62,9 @@ void seq_qk_norm_store(int, const void*, int, const float*, const float*, void*,
                        int, int, int, int, float, SeqDesc, hipStream_t);
 void seq_gqa_attention(int, const void*, int, const void*, int, const void*, int, float*, float*, float*, const float*,
                        int, int, int, int, float, const float*, void*, int, float, float, const void*, int, int, int, int,
-                       int, int, int, float, const int*, const int*, int, SeqDesc, hipStream_t);
+                       int, int, int, int, float, const int*, const int*, int, SeqDesc, hipStream_t);
 void seq_rope_kv_store(int, const void*, int, const float*, void*, void*, void*, int, int, int, int, int, int, float, int,
-                       int, float, int, float, int, SeqDesc, hipStream_t);
+                       int, float, int, float, int, float, const void*, float, SeqDesc, hipStream_t);
 void seq_residual_dyt(int, int, const float*, const void*, int, float, float*, int, const float*, float*, const float*,
                       const float*, float, const float*, int, const float*, float*, void*, int, const int*, const int*, int,
                       SeqDesc, hipStream_t);
@@ -484,6 +485,27 @@ Tensor scaled_postnorm(Tensor x, Tensor y, Tensor w, double alpha, double eps, b
   return h;
 }
 
+// x (float, in place) <- x + rms(y) * w; returns its copy in the activation type or, with wn, rms(x) * wn
+Tensor residual_postnorm(Tensor x, Tensor y, Tensor w, double eps, bool out_bf16, optional<Tensor> wn) {
+  f32c(x, "x");
+  f32c(w, "w");
+  const int W = (int)x.size(-1), T = (int)(x.numel() / W), code = out_bf16 ? 0 : 1;
+  const bool yf = y.scalar_type() == at::kFloat;
+  TORCH_CHECK(w.numel() == W, "norm weight size");
+  TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.size(0) == T && y.size(1) == W && (T == 0 || y.stride(1) == 1) &&
+                  (yf || code_of(y) == code), "y: [T, W], float or the activation type");
+  const float* np = nullptr;
+  if (wn && wn->defined()) {
+    f32c(*wn, "next norm weight");
+    TORCH_CHECK(wn->numel() == W, "next norm weight size");
+    np = wn->data_ptr<float>();
+  }
+  auto h = at::empty({T, W}, x.options().dtype(out_bf16 ? at::kBFloat16 : at::kFloat));
+  seq_residual_postnorm(code, yf ? 1 : 0, x.data_ptr<float>(), y.data_ptr(), ld(y), w.data_ptr<float>(), np, h.data_ptr(), T,
+                        W, (float)eps, stream());
+  return h;
+}
+
 Tensor rms_act(Tensor u, Tensor w, double eps) {
   const int code = code_of(u);
   TORCH_CHECK(u.dim() == 2, "u: [T, n]");
@@ -594,8 +616,8 @@ Tensor latent_attention(Tensor qa, Tensor q, Tensor cache, optional<Tensor> gate
     auto pm = at::empty({np, H, nsplit}, fo), pl = at::empty({np, H, nsplit}, fo), pu = at::empty({np, H, nsplit, R}, fo);
     seq_gqa_attention(code, Q.data_ptr(), (int)(H * (R + dr)), cache.data_ptr(), (int)(R + dr), cache.data_ptr(),
                       (int)(R + dr), pm.data_ptr<float>(), pl.data_ptr<float>(), pu.data_ptr<float>(), nullptr, 0, 0,
-                      (int)window, has_sinks ? 1 : 0, 0.f, sp, out.data_ptr(), (int)(H * R), 1.f, 0.f, nullptr, 0, (int)H, 1,
-                      (int)(R + dr),
+                      (int)window, has_sinks ? 1 : 0, 0.f, sp, out.data_ptr(), (int)(H * R), 1.f, 0.f, nullptr, 0, 0, (int)H,
+                      1, (int)(R + dr),
                       (int)R, (int)cache.size(1), (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
     return out;
   }
@@ -624,7 +646,7 @@ static const float* check_routing(int64_t n, const optional<Tensor>& corr, int64
 
 std::vector<Tensor> route_grouped(Tensor z, optional<Tensor> corr, int64_t top, int64_t groups, int64_t keep,
                                   double scale, int64_t kind) {
-  TORCH_CHECK(kind >= 0 && kind < 8, "routing kind");
+  TORCH_CHECK(kind >= 0 && kind < 16, "routing kind");
   f32c(z, "router logits");
   TORCH_CHECK(z.dim() == 2, "router logits: [T, n]");
   const int64_t T = z.size(0), n = z.size(1);
@@ -640,7 +662,7 @@ std::vector<Tensor> route_grouped(Tensor z, optional<Tensor> corr, int64_t top, 
 // the last `extra` router rows are not routed: their products come back as a third tensor, float [T, extra]
 std::vector<Tensor> route_fused(Tensor h, Tensor router, optional<Tensor> corr, int64_t top, int64_t groups,
                                 int64_t keep, double scale, int64_t kind, int64_t extra) {
-  TORCH_CHECK(kind >= 0 && kind < 8, "routing kind");
+  TORCH_CHECK(kind >= 0 && kind < 16, "routing kind");
   const int code = code_of(h);
   TORCH_CHECK(h.dim() == 2, "h: [T, W]");
   const int64_t T = h.size(0), W = h.size(1);
@@ -832,7 +854,7 @@ Tensor qk_norm_store(Tensor u, int64_t nq, int64_t nk, Tensor qw, Tensor kw, Ten
 Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, int64_t H, int64_t G, double scale,
                         int64_t block, bool sink, double sink_logit, int64_t nsplit, std::vector<Tensor> desc,
                         std::vector<Tensor> tiles, int64_t window, optional<Tensor> sinks, optional<Tensor> out_,
-                        double out_scale, double softcap, optional<Tensor> gate) {
+                        double out_scale, double softcap, optional<Tensor> gate, int64_t keep_first) {
   const int code = code_of(q);
   TORCH_CHECK(q.dim() == 2 && H >= 1 && G >= 1 && H % G == 0 && q.size(1) % H == 0, "q: [T, H * dk]");
   const int64_t T = q.size(0), dk = q.size(1) / H;
@@ -843,6 +865,9 @@ Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, i
   const int64_t dv = vc.size(2) / G, max_len = kc.size(1);
   TORCH_CHECK(dv >= 1 && dv <= seq_attn_max_cols(), "attention: dv above ", seq_attn_max_cols());
   TORCH_CHECK(nsplit >= 1 && nsplit <= 1024 && block >= 0 && window >= 0, "nsplit, block, window");
+  TORCH_CHECK(keep_first >= 0 && keep_first <= (1 << 30), "keep_first");
+  TORCH_CHECK(keep_first == 0 || (window > 0 && block == 0 && !(bias && bias->defined())),
+              "kept first keys go with a window, without blocks or a bias");
   const float* sp = nullptr;
   if (sinks && sinks->defined()) {
     f32c(*sinks, "sinks");
@@ -896,16 +921,17 @@ Tensor biased_attention(Tensor q, Tensor kc, Tensor vc, optional<Tensor> bias, i
   auto pu = at::empty({np, H, nsplit, dv}, fo);
   seq_gqa_attention(code, q.data_ptr(), ld(q), kc.data_ptr(), (int)(G * dk), vc.data_ptr(), (int)(G * dv),
                     pm.data_ptr<float>(), pl.data_ptr<float>(), pu.data_ptr<float>(), bp, nd, (int)block, (int)window,
-                    sink ? 1 : 0, (float)sink_logit, sp, out.data_ptr(), ldo, (float)out_scale, (float)softcap, gp, ldg, (int)H,
-                    (int)G, (int)dk, (int)dv, (int)max_len, (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
+                    sink ? 1 : 0, (float)sink_logit, sp, out.data_ptr(), ldo, (float)out_scale, (float)softcap, gp, ldg,
+                    (int)keep_first, (int)H, (int)G, (int)dk, (int)dv, (int)max_len, (int)nsplit, (float)scale, tseq, tt0, ntiles, d, stream());
   return out;
 }
 
 // u [T, nq + nk (+ nv)]: rotated q returned, rotated k and the values (u's v columns, or the k columns as they came) go
-// to the caches at each token's (slot, position)
+// to the caches at each token's (slot, position).  qk_eps >= 0: rotated q and k heads are divided by their root mean
+// square; v_first: the values are blended with that cache's, (1 - lam) v + lam v_first
 Tensor rope_kv_store(Tensor u, int64_t nq, int64_t nk, int64_t H, int64_t G, Tensor inv_freq, int64_t dims, Tensor kc,
                      Tensor vc, std::vector<Tensor> desc, bool half, double mag, bool values_are_keys, double temp_coef,
-                     int64_t temp_every, double v_eps) {
+                     int64_t temp_every, double v_eps, double qk_eps, optional<Tensor> v_first, double lam) {
   const int code = code_of(u);
   TORCH_CHECK(u.dim() == 2 && H >= 1 && G >= 1 && nq % H == 0 && nk % G == 0 && nq / H == nk / G &&
                   u.size(1) >= nq + nk, "u: [T, H * dk + G * dk (+ nv)]");
@@ -917,11 +943,20 @@ Tensor rope_kv_store(Tensor u, int64_t nq, int64_t nk, int64_t H, int64_t G, Ten
   check_kv_cache(kc, nk, code, "key cache");
   check_kv_cache(vc, nv, code, "value cache");
   TORCH_CHECK(vc.size(0) == kc.size(0) && vc.size(1) == kc.size(1), "caches: one pool of slots");
+  TORCH_CHECK(dims <= 8192, "rotated dimensions above 8192");
+  const void* fp = nullptr;
+  if (v_first && v_first->defined()) {
+    check_kv_cache(*v_first, nv, code, "first value cache");
+    TORCH_CHECK(v_first->sizes() == vc.sizes() && !values_are_keys && v_eps < 0,
+                "first value cache: the value cache's shape, plain values");
+    fp = v_first->data_ptr();
+  }
   SeqDesc d = desc_of(desc, optional<Tensor>(), T);
   auto q = at::empty({T, nq}, u.options());
   seq_rope_kv_store(code, u.data_ptr(), ld(u), inv_freq.data_ptr<float>(), q.data_ptr(), kc.data_ptr(), vc.data_ptr(),
                     (int)nq, (int)nk, (int)nv, (int)dk, (int)dims, half ? 1 : 0, (float)mag, values_are_keys ? 1 : 0,
-                    (int)kc.size(1), (float)temp_coef, (int)temp_every, (float)v_eps, (int)(nv / G), d, stream());
+                    (int)kc.size(1), (float)temp_coef, (int)temp_every, (float)v_eps, (int)(nv / G), (float)qk_eps,
+                    fp, (float)lam, d, stream());
   return q;
 }
 
@@ -1157,6 +1192,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_pair", &embed_pair, py::arg("tok"), py::arg("table"), py::arg("pair"), py::arg("prev"), py::arg("scale"),
         py::arg("mul_prev"), py::arg("mul_cur"), py::arg("desc"), py::arg("live"), py::arg("out") = py::none());
   m.def("scaled_postnorm", &scaled_postnorm);
+  m.def("residual_postnorm", &residual_postnorm);
   m.def("rms_act", &rms_act);
   m.def("gate_group_norm", &gate_group_norm);
   m.def("latent_kv_store", &latent_kv_store);

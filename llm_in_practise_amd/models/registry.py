@@ -40,6 +40,11 @@ def _vefunex():
     return VefunexForCausalLM
 
 
+def _tiburax():
+    from .tiburax import TiburaxForCausalLM
+    return TiburaxForCausalLM
+
+
 REGISTRY = {
     "qwen3": _qwen, "qwen2": _qwen, "qwen3forcausallm": _qwen, "qwen2forcausallm": _qwen,
     "mobupel": _mobupel, "mobupelforcausallm": _mobupel,
@@ -47,6 +52,7 @@ REGISTRY = {
     "kitonex": _kitonex, "kitonexforcausallm": _kitonex,
     "mamivik": _mamivik, "mamivikforcausallm": _mamivik,
     "vefunex": _vefunex, "vefunexforcausallm": _vefunex,
+    "tiburax": _tiburax, "tiburaxforcausallm": _tiburax,
 }
 
 

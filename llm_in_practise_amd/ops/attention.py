@@ -262,26 +262,34 @@ def qk_norm_store(u: torch.Tensor, nq: int, nk: int, q_weight: torch.Tensor, k_w
 
 def rope_kv_store(u: torch.Tensor, nq: int, nk: int, heads: int, kv_heads: int, inv_freq: torch.Tensor, rot_dims: int,
                   k_cache: torch.Tensor, v_cache: torch.Tensor, sb, half: bool = True, mag: float = 1.0,
-                  values_are_keys: bool = False, temp: tuple | None = None, v_eps: float | None = None) -> torch.Tensor:
+                  values_are_keys: bool = False, temp: tuple | None = None, v_eps: float | None = None,
+                  qk_eps: float | None = None, v_first: tuple | None = None) -> torch.Tensor:
     """The step's ``[q | k (| v)]`` rows ``u`` on their way into rotary attention: the first ``rot_dims`` entries of
     every q and k head are rotated at the token's position (``half``: entries ``i, i + rot_dims/2`` form a pair, else
     neighbours; ``mag`` multiplies sine and cosine); the rotated k goes to ``k_cache`` ``[slots, max_len, nk]`` at each
     token's slot and position; ``v_cache`` gets ``u``'s v columns or, with ``values_are_keys``, the k columns as they
     came (unrotated).  Angles and the rotation are float.  Returns the rotated q ``[T, nq]``.  ``temp = (coef, every)``:
     q at position ``p`` is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``.  ``v_eps``: each kv head's value
-    is divided by its root mean square (that eps inside the root) before it is cached.  ``rot_dims = 0``: no rotation."""
+    is divided by its root mean square (that eps inside the root) before it is cached.  ``rot_dims = 0``: no rotation.
+    ``qk_eps``: every rotated q and k head is divided by its root mean square (that eps inside the root).
+    ``v_first = (cache, lam)``: the values are cached as ``(1 - lam) v + lam cache[slot, pos]``, the blend with another
+    layer's values of the same token (plain values only)."""
     from ._native import native_seq, use_seq
+    if v_first is not None and (values_are_keys or v_eps is not None):
+        raise ValueError("rope_kv_store: only plain values are blended with another layer's")
     if use_seq(u):
+        first, lam = v_first or (None, 0.0)
         return native_seq().rope_kv_store(u, nq, nk, heads, kv_heads, inv_freq, rot_dims, k_cache, v_cache, sb.desc, half,
-                                          mag, values_are_keys, *(temp or (0.0, 0)), -1.0 if v_eps is None else v_eps)
+                                          mag, values_are_keys, *(temp or (0.0, 0)), -1.0 if v_eps is None else v_eps,
+                                          -1.0 if qk_eps is None else qk_eps, first, lam)
     return ref.rope_kv_store(u, nq, nk, heads, kv_heads, inv_freq, rot_dims, k_cache, v_cache, sb, half, mag,
-                             values_are_keys, temp, v_eps)
+                             values_are_keys, temp, v_eps, qk_eps, v_first)
 
 
 def biased_attention(q, k_cache, v_cache, bias: torch.Tensor | None, heads: int, kv_heads: int, scale: float, sb,
                      block: int = 0, sink: float | torch.Tensor | None = None, nsplit: int = 1, window: int = 0,
                      out: torch.Tensor | None = None, out_scale: float = 1.0, softcap: float = 0.0,
-                     gate: torch.Tensor | None = None):
+                     gate: torch.Tensor | None = None, keep_first: int = 0):
     """Causal grouped-query softmax attention over a slot-indexed cache with optional parts:
     ``bias`` float ``[H, ND]`` adds ``bias[h, min(i - j, ND - 1)]`` to the scaled score of query ``i`` and key ``j``
     (``scale`` does not multiply it); ``block > 0`` lets a query see only keys of its own run of ``block`` positions
@@ -293,12 +301,16 @@ def biased_attention(q, k_cache, v_cache, bias: torch.Tensor | None, heads: int,
     back (itself included).  ``out`` (``[T, H*dv]``, a column slice of a wider matrix is fine) receives the result,
     multiplied by ``out_scale``.  ``softcap > 0``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` (before
     a bias; a sink is not capped).  ``gate`` ``[T, H*dv]`` (a column slice is fine): the result is multiplied element by
-    element with its sigmoid."""
+    element with its sigmoid.  ``keep_first > 0`` (with a window, without blocks or a bias): the keys of a sequence's first
+    ``keep_first`` positions stay visible from any distance; sweeps read them and the window and nothing between."""
     from ._native import native_seq, use_seq
+    if keep_first and (window <= 0 or block or bias is not None):
+        raise ValueError("biased_attention: kept first keys go with a window, without blocks or a bias")
     if use_seq(q):
         per_head = sink if torch.is_tensor(sink) else None
         return native_seq().biased_attention(q, k_cache, v_cache, bias, heads, kv_heads, scale, block,
                                              sink is not None, 0.0 if per_head is not None else float(sink or 0.0),
-                                             nsplit, sb.desc, sb.tiles, window, per_head, out, out_scale, softcap, gate)
+                                             nsplit, sb.desc, sb.tiles, window, per_head, out, out_scale, softcap, gate,
+                                             keep_first)
     return ref.biased_attention(q, k_cache, v_cache, bias, heads, kv_heads, scale, block, sink, sb, window, out, out_scale,
-                                softcap, gate)
+                                softcap, gate, keep_first)

@@ -138,50 +138,55 @@ def moe_combine(ys: torch.Tensor, d: Dispatch, w: torch.Tensor, base: torch.Tens
 
 
 # ------------------------------------------------------------------ serving: grouped routing, identity experts
-ROUTE_SIGMOID, ROUTE_TOP2, ROUTE_NORMALIZE = 1, 2, 4
+ROUTE_SIGMOID, ROUTE_TOP2, ROUTE_NORMALIZE, ROUTE_BIAS = 1, 2, 4, 8
 
 
-def _route_kind(score: str, group_rank: str, normalize: bool) -> int:
+def _route_kind(score: str, group_rank: str, normalize: bool, correction=None, bias=None) -> int:
     if score not in ("softmax", "sigmoid") or group_rank not in ("max", "top2"):
         raise ValueError(f"routing: unknown score {score!r} or group rank {group_rank!r}")
-    return (ROUTE_SIGMOID if score == "sigmoid" else 0) | (ROUTE_TOP2 if group_rank == "top2" else 0) | \
+    if bias is not None and correction is not None:
+        raise ValueError("routing: a bias of the logits is not combined with a selection-only correction")
+    return (ROUTE_BIAS if bias is not None else 0) | (ROUTE_SIGMOID if score == "sigmoid" else 0) | (ROUTE_TOP2 if group_rank == "top2" else 0) | \
         (ROUTE_NORMALIZE if normalize else 0)
 
 
 def route_grouped(logits: torch.Tensor, correction: torch.Tensor | None, top: int, groups: int = 1, keep: int = 1,
-                  scale: float = 1.0, score: str = "softmax", group_rank: str = "max", normalize: bool = False):
+                  scale: float = 1.0, score: str = "softmax", group_rank: str = "max", normalize: bool = False,
+                  bias: torch.Tensor | None = None):
     """Float router logits ``[T, n]`` -> ``(expert ids int32 [T, top], weights float [T, top])``.  Scores are the
     softmax over all ``n`` outputs (``score="sigmoid"``: each output's own sigmoid); the choice is made on
     ``score + correction``, restricted to the ``keep`` best of ``groups`` equal runs of neighbouring outputs (a run's
     rank is its largest choice value, or with ``group_rank="top2"`` the sum of its two largest); the weights are the
-    plain scores times ``scale``, with ``normalize`` first divided by their sum over the chosen (+ 1e-20)."""
+    plain scores times ``scale``, with ``normalize`` first divided by their sum over the chosen (+ 1e-20).  ``bias`` float
+    ``[n]`` is added to the logits, so that scores, choice and weights all see it (with ``normalize`` and the softmax: the
+    softmax over the chosen biased logits); not together with a correction."""
     from . import reference as ref
     from ._native import native_seq, use_seq
-    kind = _route_kind(score, group_rank, normalize)
+    kind = _route_kind(score, group_rank, normalize, correction, bias)
     if use_seq(logits):
-        idx, w = native_seq().route_grouped(logits.contiguous(), correction, top, groups, keep, scale, kind)
+        idx, w = native_seq().route_grouped(logits.contiguous(), correction if bias is None else bias, top, groups, keep, scale, kind)
         return idx, w
     return ref.route_scored(logits, correction, top, groups, keep, scale, score == "sigmoid", group_rank == "top2",
-                            normalize)
+                            normalize, bias)
 
 
 def route_tokens(h: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, top: int, groups: int = 1,
                  keep: int = 1, scale: float = 1.0, score: str = "softmax", group_rank: str = "max",
-                 normalize: bool = False, extra: int = 0):
+                 normalize: bool = False, extra: int = 0, bias: torch.Tensor | None = None):
     """:func:`route_grouped` on the logits ``h @ router^T`` (``router`` float ``[n, W]``; the products accumulate in
     float whatever ``h``'s dtype).  On the GPU product and routing are one kernel.  The last ``extra`` rows of
     ``router`` are not routed: their products come back raw as a third result, float ``[T, extra]`` (small per-token
     gates that read the same input ride along)."""
     from . import reference as ref
     from ._native import native_seq, use_seq
-    kind = _route_kind(score, group_rank, normalize)
+    kind = _route_kind(score, group_rank, normalize, correction, bias)
     if use_seq(h):
-        idx, w, ex = native_seq().route_fused(h, router, correction, top, groups, keep, scale, kind, extra)
+        idx, w, ex = native_seq().route_fused(h, router, correction if bias is None else bias, top, groups, keep, scale, kind, extra)
         return (idx, w, ex) if extra else (idx, w)
     z = h.float() @ router.t()
     n = router.shape[0] - extra
     idx, w = ref.route_scored(z[:, :n], correction, top, groups, keep, scale, score == "sigmoid", group_rank == "top2",
-                              normalize)
+                              normalize, bias)
     return (idx, w, z[:, n:].contiguous()) if extra else (idx, w)
 
 

@@ -172,6 +172,17 @@ def scaled_postnorm(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, alph
     return ref.scaled_postnorm(x, y, weight, alpha, eps, dtype)
 
 
+def residual_postnorm(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, dtype: torch.dtype,
+                      next_weight: torch.Tensor | None = None) -> torch.Tensor:
+    """The exit of a sublayer whose output is normed, in place on the float residual: ``x <- x + rmsnorm(y) * weight``
+    (``y`` float or the activation dtype); returns ``x`` in the activation ``dtype`` (the next sublayer reads the residual
+    itself) or, with ``next_weight``, ``rmsnorm(x) * next_weight`` (the model's last norm)."""
+    from ._native import native_seq, use_seq
+    if use_seq(x):
+        return native_seq().residual_postnorm(x, y, weight, eps, dtype == torch.bfloat16, next_weight)
+    return ref.residual_postnorm(x, y, weight, eps, dtype, next_weight)
+
+
 def rms_norm_act(u: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
     """RMS norm of activation rows ``[T, n]`` (a column slice of a wider matrix is fine), statistics in float."""
     from ._native import native_seq, use_seq

@@ -323,6 +323,11 @@ def scaled_postnorm(x, y, w, alpha: float, eps: float, dtype):
     return x.to(dtype)
 
 
+def residual_postnorm(x, y, w, eps: float, dtype, next_weight=None):
+    x += _unit_rms(y.float(), eps) * w
+    return (x if next_weight is None else _unit_rms(x, eps) * next_weight).to(dtype, copy=True)
+
+
 def rms_act(u, w, eps: float):
     return (_unit_rms(u.float(), eps) * w).to(u.dtype)
 
@@ -479,7 +484,7 @@ def qk_norm_store(u, nq: int, nk: int, qw, kw, kc, vc, v_first, lam, eps: float,
 
 
 def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, sink, sb, window: int = 0, out=None,
-                     out_scale: float = 1.0, softcap: float = 0.0, gate=None):
+                     out_scale: float = 1.0, softcap: float = 0.0, gate=None, keep_first: int = 0):
     T = q.shape[0]
     dk, dv = q.shape[1] // H, vc.shape[2] // G
     rep = H // G
@@ -500,7 +505,7 @@ def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, 
         if block > 0:
             vis &= (qp[:, None] // block) == (kp[None, :] // block)
         if window > 0:
-            vis &= dist < window
+            vis &= (dist < window) | (kp[None, :] < keep_first)
         if bias is not None:
             sc = sc + bias[:, dist.clamp(0, bias.shape[1] - 1)]
         w = _softmax_with_sink(sc.masked_fill(~vis[None], float("-inf")), sink)
@@ -515,8 +520,11 @@ def biased_attention(q, kc, vc, bias, H: int, G: int, scale: float, block: int, 
     return out
 
 
-def route_scored(z, corr, top: int, groups: int, keep: int, scale: float, sigmoid: bool, top2: bool, normalize: bool):
+def route_scored(z, corr, top: int, groups: int, keep: int, scale: float, sigmoid: bool, top2: bool, normalize: bool,
+                 bias=None):
     T, n = z.shape
+    if bias is not None:
+        z = z.float() + bias
     s = torch.sigmoid(z.float()) if sigmoid else torch.softmax(z.float(), -1)
     ch = s + corr if corr is not None else s.clone()
     if groups > 1 and keep < groups:
@@ -542,18 +550,22 @@ def silu_glu(z, row_scale=None):
 
 # ---- sliding-window attention whose values are its keys, generalised delta rule, GELU GLU, element-wise output gate
 def rope_kv_store(u, nq: int, nk: int, H: int, G: int, inv_freq, dims: int, kc, vc, sb, half: bool, mag: float,
-                  values_are_keys: bool, temp=None, v_eps=None):
+                  values_are_keys: bool, temp=None, v_eps=None, qk_eps=None, v_first=None):
     T = u.shape[0]
     dk = nq // H
     pos = sb.desc[4]
-    q = rotate(u[:, :nq].float().view(T, H, dk), pos, inv_freq, dims, half, mag).reshape(T, nq)
+    norm = (lambda x: x) if qk_eps is None else (lambda x: _unit_rms(x, qk_eps))
+    q = norm(rotate(u[:, :nq].float().view(T, H, dk), pos, inv_freq, dims, half, mag)).reshape(T, nq)
     if temp is not None:
         q = q * (1.0 + temp[0] * torch.log((torch.div(pos + 1, int(temp[1]), rounding_mode="floor") + 1).float()))[:, None]
     q = q.to(u.dtype)
-    k = rotate(u[:, nq:nq + nk].float().view(T, G, dk), pos, inv_freq, dims, half, mag).reshape(T, nk)
+    k = norm(rotate(u[:, nq:nq + nk].float().view(T, G, dk), pos, inv_freq, dims, half, mag)).reshape(T, nk)
     v = u[:, nq:nq + nk] if values_are_keys else u[:, nq + nk:]
     if v_eps is not None:
         v = _unit_rms(v.float().reshape(T, G, -1), v_eps).reshape(T, -1)
+    if v_first is not None:
+        first, lam = v_first
+        v = (1.0 - lam) * v.float() + lam * first.view(-1, first.shape[2])[sb.cache_idx].float()
     kc.view(-1, nk).index_copy_(0, sb.cache_idx, k.to(kc.dtype))
     vc.view(-1, vc.shape[2]).index_copy_(0, sb.cache_idx, v.to(vc.dtype))
     return q
