@@ -225,16 +225,17 @@ def main():
                          "line is printed with '<record>': {'error': ...} and the process exits 0 "
                          "(default: 240 s, 420 s for the zero3 sub-record, which builds its own model)")
     ap.add_argument("--workload", default="train", choices=["train", "hybrid-serve", "dogudra-serve", "kitonex-serve", "mamivik-serve",
-                                                               "vefunex-serve"],
+                                                               "vefunex-serve", "tiburax-serve"],
                     help="train (default): the headline fine-tuning step.  hybrid-serve: prefill / decode tokens/s of "
                          "the Mobupel hybrid beside Qwen3 at equal size through the serving engine (one GPU); "
                          "dogudra-serve: the same for the Dogudra design beside Mobupel and Qwen3; "
                          "kitonex-serve: the same for the Kitonex design beside Dogudra and Qwen3; "
                          "mamivik-serve: the same for the Mamivik design beside Mobupel and Qwen3; "
                          "vefunex-serve: the same for the Vefunex design beside Dogudra and Qwen3; "
+                         "tiburax-serve: the same for the Tiburax design beside Vefunex and Qwen3; "
                          "--sizes / --serve-batch / --serve-prompt / --serve-decode-steps shape both")
     ap.add_argument("--serve-models", default=None,
-                    help="dogudra-serve / kitonex-serve / mamivik-serve / vefunex-serve: which of the three models to time (default: all)")
+                    help="dogudra-serve / kitonex-serve / mamivik-serve / vefunex-serve / tiburax-serve: which of the three models to time (default: all)")
     ap.add_argument("--sizes", default="w1024,w2048")
     ap.add_argument("--serve-batch", type=int, default=8)
     ap.add_argument("--serve-prompt", type=int, default=1024)
@@ -268,6 +269,12 @@ def main():
         print(json.dumps(vefunex_run(tuple(args.sizes.split(",")), args.serve_batch, args.serve_prompt,
                                      args.serve_decode_steps,
                                      models=tuple((args.serve_models or "vefunex,dogudra,qwen3").split(",")))), flush=True)
+        return
+    if args.workload == "tiburax-serve":
+        from llm_in_practise_amd.bench.tiburax_serve import run as tiburax_run
+        print(json.dumps(tiburax_run(tuple(args.sizes.split(",")), args.serve_batch, args.serve_prompt,
+                                     args.serve_decode_steps,
+                                     models=tuple((args.serve_models or "tiburax,vefunex,qwen3").split(",")))), flush=True)
         return
     from llm_in_practise_amd.ops import gemm as _lin
     if args.nf4_gemm is not None:        # else the LIPA_NF4_GEMM environment choice stands

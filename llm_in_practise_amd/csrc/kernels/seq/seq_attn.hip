@@ -440,6 +440,9 @@ static bool sweep(int code, const void* q, int ldq, const void* kc, int ldk, con
       if (x.bias == nullptr && dk == dv && (dk == 64 || dk == 96 || dk == 128)) {
         if (dk == 64) SEQ_ATTN_EXACT(4, 2); else if (dk == 96) SEQ_ATTN_EXACT(6, 3); else SEQ_ATTN_EXACT(8, 4);
         done = true;
+      } else if (x.bias == nullptr && ((dk == 96 && dv == 64) || (dk == 192 && dv == 128))) {
+        if (dk == 96) SEQ_ATTN_EXACT(6, 2); else SEQ_ATTN_EXACT(12, 4);
+        done = true;
       } else if (dk <= 64 && dv <= 64) {           // small heads: half the accumulators, more waves per SIMD
         SEQ_ATTN_FORMS(4, 2, false, false);
         done = true;
