@@ -28,10 +28,11 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 // One wave routes one token from its n router logits z (global or LDS).  s = softmax(z) over all n outputs;
 // choice = s + corr; the n outputs form `groups` equal runs of neighbours, a group's score is its largest choice and
 // only the `keep` best groups stay eligible; the `top` largest eligible choices are taken and weighted by s * scale
-// (s without the correction, not renormalised).
+// (s without the correction, not renormalised).  `always` more ids n, n + 1, .. of weight 1 follow the chosen ones (experts
+// that every token uses).
 __device__ __forceinline__ void route_wave(const float* z, const float* __restrict__ corr, int* __restrict__ idx,
                                            float* __restrict__ wout, int lane, int n, int top, int groups, int keep,
-                                           float scale, int kind) {
+                                           float scale, int kind, int always) {
   float s[RPL], ch[RPL];
   float mx = -INFINITY;
 #pragma unroll
@@ -153,6 +154,9 @@ __device__ __forceinline__ void route_wave(const float* z, const float* __restri
   if (lane < top) {
     idx[lane] = myid;
     wout[lane] = ((kind & 4) ? myw / (tot + 1e-20f) : myw) * scale;
+  } else if (lane < top + always) {
+    idx[lane] = n + lane - top;
+    wout[lane] = 1.f;
   }
 }
 
@@ -163,7 +167,7 @@ __global__ __launch_bounds__(256) void k_route_grouped(const float* __restrict__
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T_) return;
   route_wave(z + (size_t)t * n, corr, idx + (size_t)t * top, wout + (size_t)t * top, lane, n, top, groups, keep, scale,
-             kind);
+             kind, 0);
 }
 
 // four entries of an activation row as floats (16-byte rows when the width allows)
@@ -182,7 +186,7 @@ __global__ __launch_bounds__(64 * NW) void k_route_fused(const T* __restrict__ h
                                                       const float* __restrict__ corr, int* __restrict__ idx,
                                                       float* __restrict__ wout, int n, int W, int top, int groups,
                                                       int keep, float scale, int kind, int extra,
-                                                      float* __restrict__ xout) {
+                                                      float* __restrict__ xout, int always) {
   // n counts all router rows; the last `extra` of them are not routed: their products go to xout [T, extra]
   __shared__ float part[64 * RPL][4];
   __shared__ float sz[64 * RPL];
@@ -224,7 +228,8 @@ __global__ __launch_bounds__(64 * NW) void k_route_fused(const T* __restrict__ h
   __syncthreads();
   for (int e = threadIdx.x; e < extra; e += 64 * NW) xout[(size_t)t * extra + e] = sz[n - extra + e];
   if (wv == 0)
-    route_wave(sz, corr, idx + (size_t)t * top, wout + (size_t)t * top, lane, n - extra, top, groups, keep, scale, kind);
+    route_wave(sz, corr, idx + (size_t)t * (top + always), wout + (size_t)t * (top + always), lane, n - extra, top, groups,
+               keep, scale, kind, always);
 }
 
 // g = min(g, limit), u = clamp(u, -limit, limit): g * sigmoid(1.702 g) * (u + 1)
@@ -332,6 +337,35 @@ __global__ __launch_bounds__(256) void k_moe_combine(const T* __restrict__ ys, c
   }
 }
 
+// The same, four columns per thread (16-byte or 8-byte accesses); a token's ids, rows and weights are read once into LDS.
+constexpr int MAXTOP = 64;
+template <typename T>
+__global__ __launch_bounds__(256) void k_moe_combine4(const T* __restrict__ ys, const long* __restrict__ pos,
+                                                      const int* __restrict__ idx, const float* __restrict__ wts,
+                                                      const T* __restrict__ h, int ldh, const T* __restrict__ shared,
+                                                      const float* __restrict__ sgate, float* __restrict__ out, int top,
+                                                      int E, int W) {
+  __shared__ const T* row[MAXTOP];
+  __shared__ float sw[MAXTOP];
+  const size_t t = blockIdx.x;
+  const float sg = sgate != nullptr ? sigmoidf_(sgate[t]) : 1.f;
+  if (threadIdx.x < top) {
+    const size_t p = t * top + threadIdx.x;
+    const int e = idx[p];
+    row[threadIdx.x] = e >= E ? h + t * ldh : e >= 0 ? ys + (size_t)pos[p] * W : nullptr;
+    sw[threadIdx.x] = wts[p];
+  }
+  __syncthreads();
+  for (int c = 4 * threadIdx.x; c < W; c += 1024) {
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (shared != nullptr) acc = load4(shared + t * W + c) * sg;
+#pragma unroll 4
+    for (int j = 0; j < top; ++j)
+      if (row[j] != nullptr) acc += load4(row[j] + c) * sw[j];
+    *reinterpret_cast<f32x4*>(out + t * W + c) = acc;
+  }
+}
+
 // feed-forward activations on a GEMM output: mode 0 tanh-form GELU of z [T, F]; mode 1 clipped GLU, mode 2 SiLU GLU,
 // mode 3 tanh-form GELU GLU of the [gate | up] halves of z [T, 2F]
 template <typename T>
@@ -361,15 +395,15 @@ void seq_route_grouped(const float* z, const float* corr, int* idx, float* w, in
 
 void seq_route_fused(int code, const void* h, int ldh, const float* router, const float* corr, int* idx, float* w,
                      int T_, int n, int W, int top, int groups, int keep, float scale, int kind, int extra, float* xout,
-                     hipStream_t st) {
+                     int always, hipStream_t st) {
   if (T_ == 0) return;
   SEQ_DISPATCH_T(code, {
     if (T_ < 256)
       hipLaunchKernelGGL((k_route_fused<T, 16>), dim3(T_), dim3(1024), 0, st, (const T*)h, ldh, router, corr, idx, w, n,
-                         W, top, groups, keep, scale, kind, extra, xout);
+                         W, top, groups, keep, scale, kind, extra, xout, always);
     else
       hipLaunchKernelGGL((k_route_fused<T, 4>), dim3(T_), dim3(256), 0, st, (const T*)h, ldh, router, corr, idx, w, n, W,
-                         top, groups, keep, scale, kind, extra, xout);
+                         top, groups, keep, scale, kind, extra, xout, always);
   });
   LIPA_CHECK_LAUNCH();
 }
@@ -391,6 +425,13 @@ void seq_moe_pairs(int code, const void* h, int ldh, const void* wgu, const void
 void seq_moe_combine(int code, const void* ys, const long* pos, const int* idx, const float* wts, const void* h, int ldh,
                      const void* shared, const float* sgate, float* out, int T_, int top, int E, int W, hipStream_t st) {
   if (T_ == 0) return;
+  const auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  if (W % 4 == 0 && ldh % 4 == 0 && top <= MAXTOP && aligned(ys) && aligned(h) && aligned(shared) && aligned(out)) {
+    SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_moe_combine4<T>, dim3(T_), dim3(256), 0, st, (const T*)ys, pos, idx, wts,
+                                            (const T*)h, ldh, (const T*)shared, sgate, out, top, E, W));
+    LIPA_CHECK_LAUNCH();
+    return;
+  }
   SEQ_DISPATCH_T(code, hipLaunchKernelGGL(k_moe_combine<T>, dim3(T_), dim3(256), 0, st, (const T*)ys, pos, idx, wts,
                                           (const T*)h, ldh, (const T*)shared, sgate, out, top, E, W));
   LIPA_CHECK_LAUNCH();

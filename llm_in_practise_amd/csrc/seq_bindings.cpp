@@ -49,7 +49,7 @@ void seq_latent_merge(int, const float*, const float*, const float*, const void*
                       hipStream_t);
 void seq_route_grouped(const float*, const float*, int*, float*, int, int, int, int, int, float, int, hipStream_t);
 void seq_route_fused(int, const void*, int, const float*, const float*, int*, float*, int, int, int, int, int, int, float,
-                     int, int, float*, hipStream_t);
+                     int, int, float*, int, hipStream_t);
 void seq_moe_pairs(int, const void*, int, const void*, const void*, const int*, const float*, const void*, const float*,
                    void*, float*, int, int, int, int, int, float, int, int, hipStream_t);
 void seq_moe_combine(int, const void*, const long*, const int*, const float*, const void*, int, const void*, const float*,
@@ -661,7 +661,7 @@ std::vector<Tensor> route_grouped(Tensor z, optional<Tensor> corr, int64_t top, 
 // the router product (float weights [n, W], activations h [T, W] as they are, float accumulation) and the routing
 // the last `extra` router rows are not routed: their products come back as a third tensor, float [T, extra]
 std::vector<Tensor> route_fused(Tensor h, Tensor router, optional<Tensor> corr, int64_t top, int64_t groups,
-                                int64_t keep, double scale, int64_t kind, int64_t extra) {
+                                int64_t keep, double scale, int64_t kind, int64_t extra, int64_t always) {
   TORCH_CHECK(kind >= 0 && kind < 16, "routing kind");
   const int code = code_of(h);
   TORCH_CHECK(h.dim() == 2, "h: [T, W]");
@@ -671,13 +671,14 @@ std::vector<Tensor> route_fused(Tensor h, Tensor router, optional<Tensor> corr, 
   TORCH_CHECK(router.dim() == 2 && router.size(1) == W, "router: [n, W]");
   const int64_t n = router.size(0);
   TORCH_CHECK(extra >= 0 && extra < n && n <= seq_route_max_outputs(), "router rows");
+  TORCH_CHECK(always >= 0 && top + always <= 64, "always-on ids");
   const float* cp = check_routing(n - extra, corr, top, groups, keep);
-  auto idx = at::empty({T, top}, h.options().dtype(at::kInt));
-  auto w = at::empty({T, top}, h.options().dtype(at::kFloat));
+  auto idx = at::empty({T, top + always}, h.options().dtype(at::kInt));
+  auto w = at::empty({T, top + always}, h.options().dtype(at::kFloat));
   auto ex = at::empty({T, extra}, h.options().dtype(at::kFloat));
   seq_route_fused(code, h.data_ptr(), ld(h), router.data_ptr<float>(), cp, idx.data_ptr<int>(), w.data_ptr<float>(),
                   (int)T, (int)n, (int)W, (int)top, (int)groups, (int)keep, (float)scale, (int)kind, (int)extra,
-                  ex.data_ptr<float>(), stream());
+                  ex.data_ptr<float>(), (int)always, stream());
   return {idx, w, ex};
 }
 

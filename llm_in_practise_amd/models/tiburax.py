@@ -251,26 +251,35 @@ class SelectiveScanMixer(_Sublayer):
 
 
 class BiasRoutedFF(_Sublayer):
-    """SiLU-GLU experts: the ``top`` largest biased logits, softmax over those; a shared expert for every token."""
+    """SiLU-GLU experts: the ``top`` largest biased logits, softmax over those; a shared expert for every token.  With few
+    tokens (decode steps) a shared expert of the others' width is one more (token, expert) pair of weight 1."""
 
     def __init__(self, mlp: dict, W: dict, p: str, dtype, dev):
         super().__init__()
         self.E, self.top = int(mlp["router"]["experts"]), int(mlp["router"]["top"])
         self.put("router", _f32(W[p + "router"], dev))
         self.put("bias", _f32(W[p + "router.b"], dev))
-        self.put("w_gu", torch.stack([torch.stack([W[f"{p}e{e}.gate"], W[f"{p}e{e}.up"]]) for e in range(self.E)])
-                 .to(device=dev, dtype=dtype).contiguous())                                  # [E, 2, F, W]
-        self.put("w_d", torch.stack([W[f"{p}e{e}.down"] for e in range(self.E)]).to(device=dev, dtype=dtype).contiguous())
         self.shared = mlp.get("shared") is not None
-        if self.shared:
+        self.pairs = self.shared and W[p + "shared.gate"].shape == W[p + "e0.gate"].shape
+        names = [f"{p}e{e}." for e in range(self.E)] + ([p + "shared."] if self.pairs else [])
+        self.put("w_gu", torch.stack([torch.stack([W[n + "gate"], W[n + "up"]]) for n in names])
+                 .to(device=dev, dtype=dtype).contiguous())                                  # [E (+ 1), 2, F, W]
+        self.put("w_d", torch.stack([W[n + "down"] for n in names]).to(device=dev, dtype=dtype).contiguous())
+        if self.shared and not self.pairs:
             self.put("ws_gu", _act(torch.cat([W[p + "shared.gate"], W[p + "shared.up"]], 0), dtype, dev))
             self.put("ws_d", _act(W[p + "shared.down"], dtype, dev))
 
+    def _shared(self, h):
+        gu, d = (self.w_gu[-1].view(-1, h.shape[1]), self.w_d[-1]) if self.pairs else (self.ws_gu, self.ws_d)
+        return silu_glu(h @ gu.t()) @ d.t()
+
     def forward(self, h, sb: SeqBatch):
-        idx, w = route_tokens(h, self.router, None, self.top, normalize=True, bias=self.bias)
-        sh = silu_glu(h @ self.ws_gu.t()) @ self.ws_d.t() if self.shared else None
         few = sb.decode or h.shape[0] * self.top <= FEW_PAIRS
-        return moe_glu_experts(h, self.w_gu, self.w_d, idx, w, 0.0, sh, few, act="silu")
+        always = int(few and self.pairs)
+        idx, w = route_tokens(h, self.router, None, self.top, normalize=True, bias=self.bias, always=always)
+        sh = self._shared(h) if self.shared and not always else None
+        E = self.E + always
+        return moe_glu_experts(h, self.w_gu[:E], self.w_d[:E], idx, w, 0.0, sh, few, act="silu")
 
 
 class TiburaxLayer(nn.Module):

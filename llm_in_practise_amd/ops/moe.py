@@ -172,21 +172,26 @@ def route_grouped(logits: torch.Tensor, correction: torch.Tensor | None, top: in
 
 def route_tokens(h: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, top: int, groups: int = 1,
                  keep: int = 1, scale: float = 1.0, score: str = "softmax", group_rank: str = "max",
-                 normalize: bool = False, extra: int = 0, bias: torch.Tensor | None = None):
+                 normalize: bool = False, extra: int = 0, bias: torch.Tensor | None = None, always: int = 0):
     """:func:`route_grouped` on the logits ``h @ router^T`` (``router`` float ``[n, W]``; the products accumulate in
     float whatever ``h``'s dtype).  On the GPU product and routing are one kernel.  The last ``extra`` rows of
     ``router`` are not routed: their products come back raw as a third result, float ``[T, extra]`` (small per-token
-    gates that read the same input ride along)."""
+    gates that read the same input ride along).  ``always``: that many more ids, following the routed ones' (``n``,
+    ``n + 1``, ..), with weight 1 end every token's lists: experts that every token uses."""
     from . import reference as ref
     from ._native import native_seq, use_seq
     kind = _route_kind(score, group_rank, normalize, correction, bias)
     if use_seq(h):
-        idx, w, ex = native_seq().route_fused(h, router, correction if bias is None else bias, top, groups, keep, scale, kind, extra)
+        idx, w, ex = native_seq().route_fused(h, router, correction if bias is None else bias, top, groups, keep, scale, kind, extra,
+                                                always)
         return (idx, w, ex) if extra else (idx, w)
     z = h.float() @ router.t()
     n = router.shape[0] - extra
     idx, w = ref.route_scored(z[:, :n], correction, top, groups, keep, scale, score == "sigmoid", group_rank == "top2",
                               normalize, bias)
+    if always:
+        ids = torch.arange(n, n + always, dtype=idx.dtype, device=idx.device)
+        idx, w = torch.cat([idx, ids.expand(len(idx), -1)], 1), torch.cat([w, w.new_ones(len(w), always)], 1)
     return (idx, w, z[:, n:].contiguous()) if extra else (idx, w)
 
 

@@ -311,11 +311,12 @@ def test_selective_scan_alone(device, kw):
 
 
 @pytest.mark.parametrize("device", DEVICES)
-@pytest.mark.parametrize("experts,top,shared", [(1, 1, 9), (5, 1, 0), (6, 2, 33), (4, 4, 8), (70, 3, 12)])
-def test_experts(device, experts, top, shared):
-    """Top 1, some and all of the experts, with and without a shared one; prompts on the pair path and (long ones) on the
-    sorted path; a bias that only moved the choice would be seen."""
-    cfg = config([mamba(mlp=moe(experts, top, 12, shared))])
+@pytest.mark.parametrize("experts,top,shared,width", [(1, 1, 9, 44), (5, 1, 0, 44), (6, 2, 33, 45), (4, 4, 8, 44), (70, 3, 12, 44), (3, 2, 12, 42)])
+def test_experts(device, experts, top, shared, width):
+    """Top 1, some and all of the experts, without a shared one, with one of its own width and of the experts' (one more
+    pair then); prompts on the pair path and (long ones) on the sorted path, rows of whole and cut 16-byte runs; a bias that
+    only moved the choice would be seen."""
+    cfg = config([mamba(mlp=moe(experts, top, 12, shared))], width=width)
     lm, W = build(cfg, device, 3)
     toks = tokens(90, cfg["vocab"], 4)
     want = logits_of(cfg, W, toks)
@@ -324,7 +325,7 @@ def test_experts(device, experts, top, shared):
     if top > 1:
         with planted(BIAS_CHOOSES_ONLY=True):
             assert err(logits_of(cfg, W, toks), want) > 1e-3
-    h = torch.randn(700, 44, generator=torch.Generator().manual_seed(1))                     # padded runs of rows
+    h = torch.randn(700, width, generator=torch.Generator().manual_seed(1))                     # padded runs of rows
     from llm_in_practise_amd.models.common import SeqBatch, SeqStateCache
     sb = SeqBatch.packed(SeqStateCache([{}], 1, 700, torch.float32, device), [0], [700])
     close(lm.model.layers[0].ff(h.to(device), sb), O.experts(W, "l0.mlp.", cfg["layers"][0]["mlp"], h.double()))
@@ -345,6 +346,9 @@ def test_router_bias(device, n, top, score):
                    route_grouped(d(h) @ d(r).t(), None, top, score=score, normalize=True, bias=d(b))):
         dense = torch.zeros(11, n, dtype=F64).scatter_(1, idx.long().cpu(), w.double().cpu())
         close(dense, torch.zeros(11, n, dtype=F64).scatter_(1, best.indices, s), 1e-4)
+    idx2, w2 = route_tokens(d(h), d(r), None, top, score=score, normalize=True, bias=d(b), always=2)
+    assert torch.equal(idx2[:, :top], route_tokens(d(h), d(r), None, top, score=score, normalize=True, bias=d(b))[0])
+    assert idx2[:, top:].tolist() == [[n, n + 1]] * 11 and bool((w2[:, top:] == 1).all())
     with pytest.raises(ValueError):
         route_tokens(d(h), d(r), d(b), top, bias=d(b))
 
