@@ -146,8 +146,8 @@ def _route_kind(score: str, group_rank: str, normalize: bool, correction=None, b
         raise ValueError(f"routing: unknown score {score!r} or group rank {group_rank!r}")
     if bias is not None and correction is not None:
         raise ValueError("routing: a bias of the logits is not combined with a selection-only correction")
-    return (ROUTE_BIAS if bias is not None else 0) | (ROUTE_SIGMOID if score == "sigmoid" else 0) | (ROUTE_TOP2 if group_rank == "top2" else 0) | \
-        (ROUTE_NORMALIZE if normalize else 0)
+    return (ROUTE_SIGMOID if score == "sigmoid" else 0) | (ROUTE_TOP2 if group_rank == "top2" else 0) | \
+        (ROUTE_NORMALIZE if normalize else 0) | (ROUTE_BIAS if bias is not None else 0)
 
 
 def route_grouped(logits: torch.Tensor, correction: torch.Tensor | None, top: int, groups: int = 1, keep: int = 1,
