@@ -14,10 +14,10 @@
 // scaled score, a block mask (a query sees only the keys of its own run of `block` positions, counted from the
 // sequence's position 0), a sliding window (a query sees only the keys less than `window` positions back, itself
 // included; the sequence's first `keep` keys may stay visible behind it), and a sink (one more key of a fixed score, or
-// of a learned score per head, without a value in every softmax).  With one key split the matrix-core sweep normalises and writes the activation type itself; otherwise
-// k_gqa_merge does.  Scores may be bounded (softcap * tanh(score / softcap)), the result may be multiplied element by
-// element with the sigmoid of a gate.  The output may be a column slice of a wider matrix (row stride ldo) and is multiplied by
-// out_scale.
+// of a learned score per head, without a value in every softmax).  With one key split the matrix-core sweep normalises
+// and writes the activation type itself; otherwise k_gqa_merge does.  Scores may be bounded (softcap * tanh(score /
+// softcap)), the result may be multiplied element by element with the sigmoid of a gate.  The output may be a column slice
+// of a wider matrix (row stride ldo) and is multiplied by out_scale.
 #include "seq_common.h"
 
 using namespace lipa;
@@ -524,8 +524,8 @@ __global__ __launch_bounds__(256) void k_gqa_merge(const float* __restrict__ pm,
 }
 
 // Grouped-query attention over a slot-indexed cache with an optional distance bias, block mask, sliding window (behind
-// which the first `keep` keys may stay visible; not with a bias) and sink.  Key rows are ldk and value rows ldv elements apart (values may be columns of the key rows: a latent cache
-// with G = 1); the output rows are ldo elements apart.
+// which the first `keep` keys may stay visible; not with a bias) and sink.  Key rows are ldk and value rows ldv elements
+// apart (values may be columns of the key rows: a latent cache with G = 1); the output rows are ldo elements apart.
 void seq_gqa_attention(int code, const void* q, int ldq, const void* kc, int ldk, const void* vc, int ldv, float* pm,
                        float* pl, float* pu, const float* bias, int nd, int block, int window, int sink, float sink_logit,
                        const float* sinks, void* out, int ldo, float out_scale, float softcap, const void* gate, int ldg,

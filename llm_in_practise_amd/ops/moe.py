@@ -164,7 +164,8 @@ def route_grouped(logits: torch.Tensor, correction: torch.Tensor | None, top: in
     from ._native import native_seq, use_seq
     kind = _route_kind(score, group_rank, normalize, correction, bias)
     if use_seq(logits):
-        idx, w = native_seq().route_grouped(logits.contiguous(), correction if bias is None else bias, top, groups, keep, scale, kind)
+        idx, w = native_seq().route_grouped(logits.contiguous(), correction if bias is None else bias, top, groups, keep,
+                                            scale, kind)
         return idx, w
     return ref.route_scored(logits, correction, top, groups, keep, scale, score == "sigmoid", group_rank == "top2",
                             normalize, bias)
@@ -182,8 +183,8 @@ def route_tokens(h: torch.Tensor, router: torch.Tensor, correction: torch.Tensor
     from ._native import native_seq, use_seq
     kind = _route_kind(score, group_rank, normalize, correction, bias)
     if use_seq(h):
-        idx, w, ex = native_seq().route_fused(h, router, correction if bias is None else bias, top, groups, keep, scale, kind, extra,
-                                                always)
+        idx, w, ex = native_seq().route_fused(h, router, correction if bias is None else bias, top, groups, keep, scale, kind,
+                                              extra, always)
         return (idx, w, ex) if extra else (idx, w)
     z = h.float() @ router.t()
     n = router.shape[0] - extra
